@@ -12,11 +12,13 @@ from .parts import stateful as _stateful_parts   # registers mixers with a state
 from .parts import gated as _gated_parts         # registers the sandwich block, attention over keys or a latent, the gated matrix memory, the depth average
 from .parts import postnorm as _postnorm_parts   # registers the postnorm block, attention with a sink, the capped feed-forward
 from .parts import differential as _differential_parts  # registers the added_norm block, attention as a difference of two maps, the forget memory
+from .parts import streams as _streams_parts     # registers the linked_streams block, the norm stored around zero, the ungated feed-forward
 from .architectures import llama as _llama       # registers LlamaForCausalLM
 from .architectures import zekalorn as _zekalorn  # registers Zekalorn
 from .architectures import fusavik as _fusavik    # registers Fusavik
 from .architectures import ruludra as _ruludra    # registers Ruludra
 from .architectures import vimilix as _vimilix    # registers Vimilix
 from .architectures import fanidra as _fanidra    # registers Fanidra
+from .architectures import fuvevik as _fuvevik    # registers Fuvevik
 
 __version__ = "0.1.0"

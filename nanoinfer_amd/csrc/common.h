@@ -231,6 +231,11 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
 // gelu in its tanh form is 0.5 g (1 + tanh y) = g sigmoid(2 y) with y = sqrt(2 / pi) (g + 0.044715 g^3).
 struct GatedUnit {
     float a = 1.f, b = 0.f;
+    bool squared = false;          // (a product without a gate) a result v is stored as relu(v)^2
+    __device__ __forceinline__ float plain(float v) const {
+        const float r = fmaxf(v, 0.f);
+        return squared ? r * r : v;
+    }
     __device__ __forceinline__ float value(float g, float u) const { return g / (1.0f + expf(-(g * (a + b * (g * g))))) * u; }
     // the same with the hardware's exp2, for results that are rounded to bfloat16
     __device__ __forceinline__ float rough(float g, float u) const { return g / (1.0f + __expf(-(g * (a + b * (g * g))))) * u; }

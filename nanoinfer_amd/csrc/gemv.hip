@@ -141,7 +141,7 @@ struct DeferArgs {
     int parts = 0;
     float eps = 0.f;
     int width = 0;                 // elements of a row of the stream
-    GatedUnit glu;                 // (gate/up epilogue) the activation of the gate
+    GatedUnit glu;                 // (gate/up epilogue) the activation of the gate; (plain store) the activation of the result
 };
 
 // The taking side: wavefront w adds up the rows w, w + WV, ... (lane l the parts l, l + 64, ...), asked for before the
@@ -373,6 +373,7 @@ __device__ __forceinline__ void skinny_finish(const floatx4_t (&acc)[NT][MB], TO
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     if constexpr (PAIRS) v[i] = defer.glu.value(a[i], b[i]);
+                    else if constexpr (EPI == EPI_STORE) v[i] = defer.glu.plain(a[i]);
                     else v[i] = a[i];
                 }
                 TOUT* dst = y + static_cast<size_t>(m) * out_width + n0;
@@ -550,6 +551,7 @@ __device__ __forceinline__ void skinny_finish(const floatx4_t (&acc)[NT][MB], TO
 #pragma unroll
             for (int w = 0; w < WV; ++w) v += red[w][ot * MB + mb][src];
             if (scaled) v *= factor_of(m);
+            if constexpr (EPI == EPI_STORE) v = defer.glu.plain(v);
         }
         TOUT* dst = y + static_cast<size_t>(m) * out_width + n;
         if constexpr (EPI == EPI_RESIDUAL) {      // float32 residual stream, this workgroup's own columns
@@ -1377,7 +1379,8 @@ static int launch_normed(const NormArgs& norm, const void* W, void* y, int M, in
 }
 
 // epilogue: 0 store in the input type, 1 store float32, 2 SwiGLU (W is [2I, K], y is [M, I]),
-// 3 add into y, the float32 residual stream [M, N] (tiled W), 4 as 2 with gelu (tanh) in silu's place.
+// 3 add into y, the float32 residual stream [M, N] (tiled W), 4 as 2 with gelu (tanh) in silu's place, 5 store relu(.)^2 in the
+// input type.
 // K must be a multiple of 16 bytes' worth of elements x 2 (bf16: 16, f32: 8); M <= 64.
 // tiled: W is in the re-tiled order described at the top (swiglu then needs N/2 to be a multiple of 16).
 // pend, n_pend (epilogue 3, at most 16 rows): float32 [n_pend, M, N] that y has not received yet and that are
@@ -1403,6 +1406,10 @@ NI_EXPORT int ni_skinny_gemm(const void* x, const void* W, void* y, int M, int N
     if (epilogue == 4) {
         defer.glu = GatedUnit::gelu_tanh();
         epilogue = 2;
+    }
+    if (epilogue == 5) {
+        defer.glu.squared = true;
+        epilogue = 0;
     }
     if (epilogue == 2 && (N % 2)) return -3;
     if (epilogue == 2 && tiled && (I % 16)) return -4;

@@ -20,10 +20,17 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
 }
 
 // ---------------------------------------------------------------- embedding: row * scale + position row
+// `freq` (float64 [(d + 1) / 2], or null): a sinusoid of the position is added, column 2i sin(position * freq[i]), column
+// 2i + 1 the cosine; the angle is a float64 product, taken to within half a turn of zero before it is rounded to float32.
+__device__ __forceinline__ void sincos_at(int position, double freq, float* sn, float* cs) {
+    const double turn = 6.283185307179586476925286766559, angle = static_cast<double>(position) * freq;
+    sincosf(static_cast<float>(angle - turn * rint(angle / turn)), sn, cs);
+}
+
 template <typename T>
 __global__ void embed_scaled_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ positions,
                                     const T* __restrict__ table, const T* __restrict__ pos_table, float* __restrict__ out,
-                                    int d, int vocab, int max_pos, float scale) {
+                                    int d, int vocab, int max_pos, float scale, const double* __restrict__ freq) {
     const int t = blockIdx.x;
     const int id = ids[t];
     if (id < 0 || id >= vocab) return;      // unreachable after the host's check
@@ -35,6 +42,19 @@ __global__ void embed_scaled_kernel(const int32_t* __restrict__ ids, const int32
         if (p < 0 || p >= max_pos) return;  // the runner refuses a request before it reaches the last position
         prow = pos_table + static_cast<size_t>(p) * d;
     }
+    if (freq) {                             // a thread takes the two columns that share an angle
+        const int p = positions[t];
+        for (int c = threadIdx.x; 2 * c < d; c += blockDim.x) {
+            float sc[2];
+            sincos_at(p, freq[c], &sc[0], &sc[1]);
+            for (int i = 2 * c; i < min(d, 2 * c + 2); ++i) {
+                float v = ld(row + i) * scale;
+                if (prow) v += ld(prow + i);
+                o[i] = v + sc[i - 2 * c];
+            }
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < d; i += blockDim.x) {
         float v = ld(row + i) * scale;
         if (prow) v += ld(prow + i);
@@ -43,14 +63,14 @@ __global__ void embed_scaled_kernel(const int32_t* __restrict__ ids, const int32
 }
 
 NI_EXPORT int ni_embed_scaled(const void* ids, const void* positions, const void* table, const void* pos_table, void* out,
-                              int T, int d, int vocab, int max_pos, float scale, int dtype, hipStream_t stream) {
+                              int T, int d, int vocab, int max_pos, float scale, const void* freq, int dtype, hipStream_t stream) {
     if (T <= 0) return 0;
     if (dtype == 0)
         embed_scaled_kernel<float><<<T, 256, 0, stream>>>((const int32_t*)ids, (const int32_t*)positions, (const float*)table,
-                                                          (const float*)pos_table, (float*)out, d, vocab, max_pos, scale);
+                                                          (const float*)pos_table, (float*)out, d, vocab, max_pos, scale, (const double*)freq);
     else
         embed_scaled_kernel<bf16_t><<<T, 256, 0, stream>>>((const int32_t*)ids, (const int32_t*)positions, (const bf16_t*)table,
-                                                           (const bf16_t*)pos_table, (float*)out, d, vocab, max_pos, scale);
+                                                           (const bf16_t*)pos_table, (float*)out, d, vocab, max_pos, scale, (const double*)freq);
     return NI_LAUNCH_RESULT();
 }
 
@@ -316,6 +336,155 @@ NI_EXPORT int ni_post_norm(void* h, const void* addends, int n_addends, float al
     return NI_LAUNCH_RESULT();
 }
 
+// ---------------------------------------------------------------- several streams around a sublayer
+// A token has S streams x_1 .. x_S of d float32 numbers.  One pass over them does what stands between two sublayers:
+//
+//   x_t <- sum_f mix[f, t] x_f + out[t] y          the sublayer that has run (mix float32 [S, S], out [S]; null: none has)
+//   u = sum_s in[s] x_s                            what the next sublayer reads (in null: the plain sum of the streams)
+//   v = u / sqrt(mean(u^2) + eps) * w              through its norm (w null: u itself)
+//
+// y is the sum of n_add float32 addends [n_add][T][d].  h holds the streams: element (t, s, c) at t * row_stride +
+// s * stream_stride + c; a stream_stride of zero is a token whose streams are all still equal, kept once.  The new streams
+// go to h_out [T][S][d] (it may be h itself; null: they are not wanted again), v to v_out [rows][d] in its type.  `rows`
+// (int32, or null): the rows of h and y to take, in this order; h_out is then null.
+// One workgroup a row.  A thread keeps the S old values of its elements in registers, so the streams are read once and
+// written once; u waits in LDS (every thread reads back its own) for the sum of squares.
+#define LINK_STREAMS_MAX 32
+
+template <typename X, int S, int V, bool EXACT>
+__global__ void link_streams_kernel(const float* h, size_t row_stride, size_t stream_stride, const float* __restrict__ y,
+                                    int n_add, size_t add_stride, const float* __restrict__ mix, const float* __restrict__ out_w,
+                                    const float* __restrict__ in_w, const float* __restrict__ w, float eps, float* h_out,
+                                    X* __restrict__ v_out, const int32_t* __restrict__ rows, int d, int s_given) {
+    extern __shared__ __attribute__((aligned(16))) float u_row[];
+    __shared__ float scratch[16];
+    const int n_s = EXACT ? S : s_given;          // EXACT: S streams; else at most S
+    const size_t t = rows ? rows[blockIdx.x] : blockIdx.x;
+    const float* src = h + t * row_stride;
+    float ss = 0.f;
+    for (int i = threadIdx.x * V; i < d; i += blockDim.x * V) {
+        float x[S][V], u[V];
+        // the loads of all streams and of the first addend are asked for before anything waits for one
+#pragma unroll
+        for (int f = 0; f < S; ++f)
+            if (EXACT || f < n_s) VecIO<float, V>::load(src + f * stream_stride + i, x[f]);
+        if (mix) {
+            float a[V];
+#pragma unroll
+            for (int e = 0; e < V; ++e) a[e] = 0.f;
+            if (n_add > 0) VecIO<float, V>::load(y + t * d + i, a);
+            for (int k = 1; k < n_add; ++k) {
+                float b[V];
+                VecIO<float, V>::load(y + k * add_stride + t * d + i, b);
+#pragma unroll
+                for (int e = 0; e < V; ++e) a[e] += b[e];
+            }
+#pragma unroll
+            for (int e = 0; e < V; ++e) u[e] = 0.f;
+#pragma unroll
+            for (int to = 0; to < S; ++to) {
+                if (!EXACT && to >= n_s) break;
+                float n[V];
+#pragma unroll
+                for (int e = 0; e < V; ++e) n[e] = 0.f;
+#pragma unroll
+                for (int f = 0; f < S; ++f) {
+                    if (!EXACT && f >= n_s) break;
+                    const float c = mix[f * n_s + to];         // (the same for every thread: a scalar)
+#pragma unroll
+                    for (int e = 0; e < V; ++e) n[e] += c * x[f][e];
+                }
+#pragma unroll
+                for (int e = 0; e < V; ++e) {
+                    n[e] += out_w[to] * a[e];
+                    u[e] += in_w ? in_w[to] * n[e] : n[e];
+                }
+                if (h_out) VecIO<float, V>::store(h_out + (t * n_s + to) * d + i, n);
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < V; ++e) u[e] = 0.f;
+#pragma unroll
+            for (int f = 0; f < S; ++f) {
+                if (!EXACT && f >= n_s) break;
+#pragma unroll
+                for (int e = 0; e < V; ++e) u[e] += in_w ? in_w[f] * x[f][e] : x[f][e];
+            }
+        }
+        if (w) {
+#pragma unroll
+            for (int e = 0; e < V; ++e) ss += u[e] * u[e];
+            VecIO<float, V>::store(u_row + i, u);
+        } else {
+            VecIO<X, V>::store(v_out + static_cast<size_t>(blockIdx.x) * d + i, u);
+        }
+    }
+    if (!w) return;
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(d) + eps);
+    for (int i = threadIdx.x * V; i < d; i += blockDim.x * V) {
+        float u[V], wv[V];
+        VecIO<float, V>::load(u_row + i, u);
+        VecIO<float, V>::load(w + i, wv);
+#pragma unroll
+        for (int e = 0; e < V; ++e) u[e] = (u[e] * inv) * wv[e];
+        VecIO<X, V>::store(v_out + static_cast<size_t>(blockIdx.x) * d + i, u);
+    }
+}
+
+struct LinkArgs {
+    const float* h; size_t row_stride, stream_stride; const float* y; int n_add; size_t add_stride;
+    const float *mix, *out_w, *in_w, *w; float eps; float* h_out; void* v_out; const int32_t* rows; int n_rows, d, s;
+};
+
+template <typename X, int S, int V, bool EXACT>
+static hipError_t launch_link(const LinkArgs& a, hipStream_t stream) {
+    const size_t lds = a.w ? static_cast<size_t>(a.d) * sizeof(float) : 0;
+    static size_t allowed = 48 * 1024;            // of this instance of the kernel
+    if (lds > allowed) {
+        const hipError_t err = hipFuncSetAttribute((const void*)link_streams_kernel<X, S, V, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (err != hipSuccess) return err;
+        allowed = lds;
+    }
+    // a thread for every piece of a row, up to 512: few rows are few workgroups, whose time is the longest chain of loads
+    const int pieces = (a.d + V - 1) / V;
+    const int threads = std::min(512, std::max(WAVE, (pieces + WAVE - 1) / WAVE * WAVE));
+    link_streams_kernel<X, S, V, EXACT><<<a.n_rows, threads, lds, stream>>>(a.h, a.row_stride, a.stream_stride, a.y, a.n_add, a.add_stride, a.mix,
+                                                                            a.out_w, a.in_w, a.w, a.eps, a.h_out, (X*)a.v_out, a.rows, a.d, a.s);
+    return hipSuccess;
+}
+
+template <typename X, int V>
+static hipError_t launch_link_streams(const LinkArgs& a, hipStream_t stream) {
+    switch (a.s) {
+        case 1: return launch_link<X, 1, V, true>(a, stream);
+        case 2: return launch_link<X, 2, V, true>(a, stream);
+        case 3: return launch_link<X, 3, V, true>(a, stream);
+        case 4: return launch_link<X, 4, V, true>(a, stream);
+        default: break;
+    }
+    if (a.s <= 8) return launch_link<X, 8, V, false>(a, stream);
+    return launch_link<X, LINK_STREAMS_MAX, 1, false>(a, stream);
+}
+
+NI_EXPORT int ni_link_streams(const void* h, int streams_in_h, const void* y, int n_add, const void* mix, const void* out_w, const void* in_w,
+                              const void* w, float eps, void* h_out, void* v_out, int v_dtype, const void* rows, int n_rows, int T, int S, int d,
+                              hipStream_t stream) {
+    if (n_rows <= 0 || T <= 0 || d <= 0) return 0;
+    if (S < 1 || S > LINK_STREAMS_MAX || (streams_in_h != 1 && streams_in_h != S) || n_add < 0 || (n_add > 0 && !y)) return -1;
+    if ((mix == nullptr) != (out_w == nullptr) || (!mix && (n_add > 0 || h_out)) || (rows && h_out) || !v_out) return -1;
+    if (!rows && n_rows != T) return -1;
+    if (w && static_cast<size_t>(d) * sizeof(float) > 150 * 1024) return -2;
+    const LinkArgs a{(const float*)h, static_cast<size_t>(streams_in_h) * d, streams_in_h == 1 ? 0 : static_cast<size_t>(d), (const float*)y, n_add,
+                     static_cast<size_t>(T) * d, (const float*)mix, (const float*)out_w, (const float*)in_w, (const float*)w, eps, (float*)h_out,
+                     v_out, (const int32_t*)rows, n_rows, d, S};
+    const bool pieces = d % 4 == 0 && aligned16(h, y) && aligned16(h_out, v_out) && aligned16(w, w);
+    hipError_t err;
+    if (v_dtype == 0) err = pieces ? launch_link_streams<float, 4>(a, stream) : launch_link_streams<float, 1>(a, stream);
+    else err = pieces ? launch_link_streams<bf16_t, 4>(a, stream) : launch_link_streams<bf16_t, 1>(a, stream);
+    if (err != hipSuccess) return (int)err;
+    return NI_LAUNCH_RESULT();
+}
+
 // ---------------------------------------------------------------- y = x / sqrt(mean(x^2) + eps) * w over columns of wider rows
 // x: n columns of float32 rows of stride `stride` (a product's accumulators); y [T, n] in the type T
 template <typename T>
@@ -560,6 +729,7 @@ NI_EXPORT int ni_rows_to_pages(const void* x, void* y, int n_pages, int page, in
 //   0  the logit; weights: the softmax among the chosen
 //   1  the logit; weights: the softmax over all E experts, not renormalised
 //   2  sigmoid(logit); weights: the values themselves, not renormalised
+//   3  the softmax over all E experts; weights: the chosen values over their sum (+ 1e-20)
 // every weight times `route_scale`.  An expert is chosen by its value plus `correction[e]` (float32 [E]; null: the value
 // alone); the weights never see the correction.
 // With `n_groups` > 1 the experts form that many equal groups of neighbours; a group counts as much as the sum of its
@@ -595,6 +765,24 @@ __global__ void route_top_kernel(const float* __restrict__ z, const float* __res
         float ze = e < E ? row[e] : -INFINITY;
         if (!(ze == ze)) ze = -INFINITY;
         raw[j] = scoring == 2 ? 1.0f / (1.0f + expf(-ze)) : ze;
+    }
+    if (scoring == 3) {             // the values are shares of all experts
+        float v = -INFINITY, sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < SLOTS; ++j) v = fmaxf(v, raw[j]);
+        v = wave_max(v);
+#pragma unroll
+        for (int j = 0; j < SLOTS; ++j) {
+            raw[j] = raw[j] > -INFINITY ? expf(raw[j] - v) : 0.f;
+            sum += raw[j];
+        }
+        sum = wave_sum(sum);
+#pragma unroll
+        for (int j = 0; j < SLOTS; ++j) raw[j] /= sum;
+    }
+#pragma unroll
+    for (int j = 0; j < SLOTS; ++j) {
+        const int e = lane + j * WAVE;
         vals[j] = e < E ? raw[j] + (correction ? correction[e] : 0.f) : -INFINITY;
     }
     if (mix_all) {                  // zeros first; the fence lets them land before lane 0 writes the chosen ones at the end
@@ -684,8 +872,9 @@ __global__ void route_top_kernel(const float* __restrict__ z, const float* __res
             best = wave_max(my_value);
             total = wave_sum(lane < top ? expf(my_value - best) : 0.f);
         }
+        if (scoring == 3) total = wave_sum(lane < top ? my_value : 0.f) + 1e-20f;
         if (lane < top) {
-            const float w = (scoring == 2 ? my_value : expf(my_value - best) / total) * route_scale;
+            const float w = (scoring == 2 ? my_value : scoring == 3 ? my_value / total : expf(my_value - best) / total) * route_scale;
             c[lane] = my_expert;
             m[lane] = w;
             if (mix_all) mix_all[static_cast<size_t>(t) * E + my_expert] = w;
@@ -699,8 +888,12 @@ __global__ void route_top_kernel(const float* __restrict__ z, const float* __res
             total = 0.f;
             for (int k = 0; k < top; ++k) total += expf(m[k] - best);
         }
+        if (scoring == 3) {
+            total = 1e-20f;
+            for (int k = 0; k < top; ++k) total += m[k];
+        }
         for (int k = 0; k < top; ++k) {
-            const float w = (scoring == 2 ? m[k] : expf(m[k] - best) / total) * route_scale;
+            const float w = (scoring == 2 ? m[k] : scoring == 3 ? m[k] / total : expf(m[k] - best) / total) * route_scale;
             m[k] = w;
             if (mix_all) mix_all[static_cast<size_t>(t) * E + c[k]] = w;
         }
@@ -724,7 +917,12 @@ route_top_lanes_kernel(const float* __restrict__ z, const float* __restrict__ co
     const bool mine = e < E;
     float ze = mine ? z[static_cast<size_t>(t) * E + e] : -INFINITY;
     if (!(ze == ze)) ze = -INFINITY;                  // a logit that is no number is never preferred
-    const float raw = scoring == 2 ? 1.0f / (1.0f + expf(-ze)) : ze;
+    float raw = scoring == 2 ? 1.0f / (1.0f + expf(-ze)) : ze;
+    if (scoring == 3) {                               // the values are shares of all experts
+        const float most = wave_max(raw);
+        raw = raw > -INFINITY ? expf(raw - most) : 0.f;
+        raw /= wave_sum(raw);
+    }
     const float val = mine ? raw + (correction ? correction[e] : 0.f) : -INFINITY;
     bool open = mine;
     if (n_groups > 1) {
@@ -752,7 +950,9 @@ route_top_lanes_kernel(const float* __restrict__ z, const float* __restrict__ co
     const bool taken = open && rank < top;
     const unsigned long long taken_mask = __ballot(taken);
     float w = raw;
-    if (scoring != 2) {
+    if (scoring == 3) {
+        w = raw / (wave_sum(taken ? raw : 0.f) + 1e-20f);
+    } else if (scoring != 2) {
         const unsigned long long over = scoring == 1 ? __ballot(mine) : taken_mask;     // what the softmax runs over
         float best = -INFINITY, total = 0.f;
         for (int j = 0; j < E; ++j)
@@ -773,7 +973,7 @@ route_top_lanes_kernel(const float* __restrict__ z, const float* __restrict__ co
 NI_EXPORT int ni_route_top(const void* z, const void* correction, void* chosen, void* mix, void* mix_all, int T, int E, int top,
                            int scoring, int n_groups, int keep, int group_top, float route_scale, hipStream_t stream) {
     if (T <= 0) return 0;
-    if (top < 1 || top > E || E > 32 * WAVE || scoring < 0 || scoring > 2 || group_top < 1) return -1;
+    if (top < 1 || top > E || E > 32 * WAVE || scoring < 0 || scoring > 3 || group_top < 1) return -1;
     if (n_groups < 1 || n_groups > WAVE || E % n_groups || keep < 1 || keep > n_groups || top > E / n_groups * keep) return -1;
     if (E <= WAVE)
         route_top_lanes_kernel<<<T, WAVE, 0, stream>>>((const float*)z, (const float*)correction, (int32_t*)chosen, (float*)mix,
@@ -789,16 +989,17 @@ NI_EXPORT int ni_route_top(const void* z, const void* correction, void* chosen, 
 
 // ---------------------------------------------------------------- all experts at once, for many rows
 // act[t, e * ff + i] = mix_all[t, e] * relu(up[t, e * ff + i])^2 : an expert that was not chosen gives
-// zeros, and the product with the experts' down matrices laid side by side is the weighted sum.
+// zeros, and the product with the experts' down matrices laid side by side is the weighted sum.  A row of mix_all has
+// `mix_stride` >= E numbers (router outputs behind the experts are somebody else's); a null mix_all: every expert counts once.
 template <typename T>
 __global__ void experts_act_kernel(const T* __restrict__ up, const float* __restrict__ mix_all, T* __restrict__ act,
-                                   int E, int ff, size_t n) {
+                                   int E, int ff, size_t n, int mix_stride) {
     const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const size_t width = static_cast<size_t>(E) * ff;
     const size_t t = i / width;
     const int e = static_cast<int>((i % width) / ff);
-    const float w = mix_all[t * E + e];
+    const float w = mix_all ? mix_all[t * mix_stride + e] : 1.f;
     float v = 0.f;
     if (w != 0.f) {
         const float u = fmaxf(ld(up + i), 0.f);
@@ -811,14 +1012,14 @@ __global__ void experts_act_kernel(const T* __restrict__ up, const float* __rest
 // expert that was not chosen are not read at all
 template <typename T>
 __global__ void experts_act_vec_kernel(const T* __restrict__ up, const float* __restrict__ mix_all, T* __restrict__ act,
-                                       int E, int ff, size_t pieces) {
+                                       int E, int ff, size_t pieces, int mix_stride) {
     const size_t idx = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (idx >= pieces) return;
     const size_t i = idx * 8;
     const size_t width = static_cast<size_t>(E) * ff;
     const size_t t = i / width;
     const int e = static_cast<int>((i - t * width) / ff);
-    const float w = mix_all[t * E + e];
+    const float w = mix_all ? mix_all[t * mix_stride + e] : 1.f;
     float v[8];
     if (w != 0.f) {
         VecIO<T, 8>::load(up + i, v);
@@ -854,13 +1055,13 @@ __device__ __forceinline__ float glu_value(float g, float u, const GluForm f) {
 // a null mix_all: every expert counts once (one feed-forward that every token uses is E = 1 of these)
 template <typename T>
 __global__ void experts_act_gated_kernel(const T* __restrict__ up, const float* __restrict__ mix_all, T* __restrict__ act,
-                                         int E, int ff, size_t n, GluForm form) {
+                                         int E, int ff, size_t n, GluForm form, int mix_stride) {
     const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const size_t width = static_cast<size_t>(E) * ff;
     const size_t t = i / width;
     const int e = static_cast<int>((i % width) / ff), c = static_cast<int>(i % ff);
-    const float w = mix_all ? mix_all[t * E + e] : 1.f;
+    const float w = mix_all ? mix_all[t * mix_stride + e] : 1.f;
     float v = 0.f;
     if (w != 0.f) {
         const T* src = up + (t * E + e) * 2 * static_cast<size_t>(ff);
@@ -873,7 +1074,7 @@ __global__ void experts_act_gated_kernel(const T* __restrict__ up, const float* 
 // expert that was not chosen are not read at all
 template <typename T>
 __global__ void experts_act_gated_vec_kernel(const T* __restrict__ up, const float* __restrict__ mix_all, T* __restrict__ act,
-                                             int E, int ff, size_t pieces, GluForm form) {
+                                             int E, int ff, size_t pieces, GluForm form, int mix_stride) {
     const size_t idx = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (idx >= pieces) return;
     const size_t i = idx * 8;
@@ -881,7 +1082,7 @@ __global__ void experts_act_gated_vec_kernel(const T* __restrict__ up, const flo
     const size_t t = i / width;
     const size_t in_row = i - t * width;
     const int e = static_cast<int>(in_row / ff), c = static_cast<int>(in_row - static_cast<size_t>(e) * ff);
-    const float w = mix_all ? mix_all[t * E + e] : 1.f;
+    const float w = mix_all ? mix_all[t * mix_stride + e] : 1.f;
     float v[8];
     if (w != 0.f) {
         const T* src = up + (t * E + e) * 2 * static_cast<size_t>(ff) + c;
@@ -898,39 +1099,39 @@ __global__ void experts_act_gated_vec_kernel(const T* __restrict__ up, const flo
 }
 
 // `gated` 0: relu(up)^2; 1: silu(gate) * up; 2: the capped form with `limit` and `slope` (see glu_value)
-NI_EXPORT int ni_experts_act(const void* up, const void* mix_all, void* act, int T, int E, int ff, int gated, float limit, float slope,
-                             int dtype, hipStream_t stream) {
+NI_EXPORT int ni_experts_act(const void* up, const void* mix_all, int mix_stride, void* act, int T, int E, int ff, int gated, float limit,
+                             float slope, int dtype, hipStream_t stream) {
     const size_t n = static_cast<size_t>(T) * E * ff;
     if (n == 0) return 0;
-    if (gated < 0 || gated > 2 || (!gated && !mix_all)) return -1;
+    if (gated < 0 || gated > 2 || (mix_all && mix_stride < E)) return -1;
     const GluForm form{gated, limit, slope};
     if (gated && ff % 8 == 0 && aligned16(up, act)) {
         const size_t pieces = n / 8;
         if (dtype == 0)
-            experts_act_gated_vec_kernel<float><<<blocks_of(pieces, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, pieces, form);
+            experts_act_gated_vec_kernel<float><<<blocks_of(pieces, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, pieces, form, mix_stride);
         else
-            experts_act_gated_vec_kernel<bf16_t><<<blocks_of(pieces, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, pieces, form);
+            experts_act_gated_vec_kernel<bf16_t><<<blocks_of(pieces, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, pieces, form, mix_stride);
         return NI_LAUNCH_RESULT();
     }
     if (gated) {
         if (dtype == 0)
-            experts_act_gated_kernel<float><<<blocks_of(n, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, n, form);
+            experts_act_gated_kernel<float><<<blocks_of(n, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, n, form, mix_stride);
         else
-            experts_act_gated_kernel<bf16_t><<<blocks_of(n, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, n, form);
+            experts_act_gated_kernel<bf16_t><<<blocks_of(n, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, n, form, mix_stride);
         return NI_LAUNCH_RESULT();
     }
     if (ff % 8 == 0 && aligned16(up, act)) {
         const size_t pieces = n / 8;
         if (dtype == 0)
-            experts_act_vec_kernel<float><<<blocks_of(pieces, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, pieces);
+            experts_act_vec_kernel<float><<<blocks_of(pieces, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, pieces, mix_stride);
         else
-            experts_act_vec_kernel<bf16_t><<<blocks_of(pieces, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, pieces);
+            experts_act_vec_kernel<bf16_t><<<blocks_of(pieces, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, pieces, mix_stride);
         return NI_LAUNCH_RESULT();
     }
     if (dtype == 0)
-        experts_act_kernel<float><<<blocks_of(n, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, n);
+        experts_act_kernel<float><<<blocks_of(n, 256), 256, 0, stream>>>((const float*)up, (const float*)mix_all, (float*)act, E, ff, n, mix_stride);
     else
-        experts_act_kernel<bf16_t><<<blocks_of(n, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, n);
+        experts_act_kernel<bf16_t><<<blocks_of(n, 256), 256, 0, stream>>>((const bf16_t*)up, (const float*)mix_all, (bf16_t*)act, E, ff, n, mix_stride);
     return NI_LAUNCH_RESULT();
 }
 
@@ -941,13 +1142,15 @@ NI_EXPORT int ni_experts_act(const void* up, const void* mix_all, void* act, int
 //   out[t, r] = sum_k mix[t, k] * W_down[r, chosen[t, k] * ff : +ff] . hid[t * top + k, :]
 // A wavefront takes R neighbouring rows at once, with a sum of its own for each: the loads of the R rows are in
 // flight together, and the input row is read once for all of them.
+// A chosen index of E or more is an identity expert: it has no matrices, its output is x[t, :] itself.
 template <typename T, int R, bool GATED>
 __global__ void experts_up_few_kernel(const T* __restrict__ x, const T* __restrict__ w_up, const int32_t* __restrict__ chosen,
-                                      float* __restrict__ hid, int d, int ff, int top, bool vec, GluForm form) {
+                                      float* __restrict__ hid, int d, int ff, int E, int top, bool vec, GluForm form) {
     // GATED: an expert owns 2 ff rows of w_up, its gate rows and then its up rows; hid = glu(gate . x, up . x)
     const int pair = blockIdx.x;                 // t * top + k
     const int t = pair / top;
     const int e = chosen[pair];
+    if (e >= E) return;                          // an identity expert has no hidden row
     const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, waves = blockDim.x / WAVE;
     const T* xr = x + static_cast<size_t>(t) * d;
     const int i0 = (blockIdx.y * waves + wave) * R;
@@ -1001,7 +1204,7 @@ __global__ void experts_up_few_kernel(const T* __restrict__ x, const T* __restri
 template <typename T, int R>
 __global__ void experts_down_few_kernel(const float* __restrict__ hid, const T* __restrict__ w_down,
                                         const int32_t* __restrict__ chosen, const float* __restrict__ mix,
-                                        float* __restrict__ out, int d, int ff, int E, int top, bool vec) {
+                                        const T* __restrict__ x, float* __restrict__ out, int d, int ff, int E, int top, bool vec) {
     const int t = blockIdx.x;
     const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, waves = blockDim.x / WAVE;
     const int r0 = (blockIdx.y * waves + wave) * R;
@@ -1012,6 +1215,12 @@ __global__ void experts_down_few_kernel(const float* __restrict__ hid, const T* 
     for (int u = 0; u < R; ++u) total[u] = 0.f;
     for (int k = 0; k < top; ++k) {
         const int e = chosen[t * top + k];
+        if (e >= E) {
+            const float weight = mix[t * top + k];
+#pragma unroll
+            for (int u = 0; u < R; ++u) total[u] += weight * ld(x + static_cast<size_t>(t) * d + min(r0 + u, d - 1));
+            continue;
+        }
         const float* hr = hid + (static_cast<size_t>(t) * top + k) * ff;
         const T* wr[R];
 #pragma unroll
@@ -1056,11 +1265,11 @@ static void launch_experts_few(const void* x, const void* w_up, const void* w_do
     constexpr int rows = 4 * R;                  // four wavefronts a workgroup
     dim3 g1(T_ * top, (ff + rows - 1) / rows), g2(T_, (d + rows - 1) / rows);
     if (gated)
-        experts_up_few_kernel<T, R, true><<<g1, 256, 0, stream>>>((const T*)x, (const T*)w_up, (const int32_t*)chosen, (float*)hid, d, ff, top, vec_up, form);
+        experts_up_few_kernel<T, R, true><<<g1, 256, 0, stream>>>((const T*)x, (const T*)w_up, (const int32_t*)chosen, (float*)hid, d, ff, E, top, vec_up, form);
     else
-        experts_up_few_kernel<T, R, false><<<g1, 256, 0, stream>>>((const T*)x, (const T*)w_up, (const int32_t*)chosen, (float*)hid, d, ff, top, vec_up, form);
+        experts_up_few_kernel<T, R, false><<<g1, 256, 0, stream>>>((const T*)x, (const T*)w_up, (const int32_t*)chosen, (float*)hid, d, ff, E, top, vec_up, form);
     experts_down_few_kernel<T, R><<<g2, 256, 0, stream>>>((const float*)hid, (const T*)w_down, (const int32_t*)chosen,
-                                                          (const float*)mix, (float*)out, d, ff, E, top, vec_down);
+                                                          (const float*)mix, (const T*)x, (float*)out, d, ff, E, top, vec_down);
 }
 
 // `gated` 0: w_up [E * ff, d], hid = relu(.)^2; 1 or 2: w_up [E * 2 ff, d] (an expert's gate rows, then its up rows),
@@ -1084,5 +1293,42 @@ NI_EXPORT int ni_experts_few(const void* x, const void* w_up, const void* w_down
         if (four) launch_experts_few<bf16_t, 4>(x, w_up, w_down, chosen, mix, hid, out, T, d, ff, E, top, g, vec_up, vec_down, stream);
         else launch_experts_few<bf16_t, 2>(x, w_up, w_down, chosen, mix, hid, out, T, d, ff, E, top, g, vec_up, vec_down, stream);
     }
+    return NI_LAUNCH_RESULT();
+}
+
+// What identity experts add in steps of many rows: out[t, :] = (sum of mix_all[t, first .. first + count)) * x[t, :], mix_all
+// float32 rows of `mix_stride`, x [T, d] in the compute type, out float32.
+template <typename T>
+__global__ void identity_experts_kernel(const T* __restrict__ x, const float* __restrict__ mix_all, int mix_stride, int first, int count,
+                                        float* __restrict__ out, int d, bool vec) {
+    const size_t t = blockIdx.x;
+    const float* m = mix_all + t * mix_stride + first;
+    float w = 0.f;
+    for (int e = 0; e < count; ++e) w += m[e];
+    const T* xr = x + t * d;
+    float* o = out + t * d;
+    if (vec) {
+        for (int i = 8 * threadIdx.x; i < d; i += 8 * blockDim.x) {
+            float v[8];
+            VecIO<T, 8>::load(xr + i, v);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] *= w;
+            VecIO<float, 8>::store(o + i, v);
+        }
+    } else {
+        for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = w * ld(xr + i);
+    }
+}
+
+NI_EXPORT int ni_identity_experts(const void* x, const void* mix_all, int mix_stride, int first, int count, void* out, int T, int d, int dtype,
+                                  hipStream_t stream) {
+    if (T <= 0 || d <= 0) return 0;
+    if (first < 0 || count < 1 || first + count > mix_stride) return -1;
+    const bool vec = d % 8 == 0 && aligned16(x, out);
+    const int threads = std::min(256, std::max(WAVE, (d / 8 + WAVE - 1) / WAVE * WAVE));
+    if (dtype == 0)
+        identity_experts_kernel<float><<<T, threads, 0, stream>>>((const float*)x, (const float*)mix_all, mix_stride, first, count, (float*)out, d, vec);
+    else
+        identity_experts_kernel<bf16_t><<<T, threads, 0, stream>>>((const bf16_t*)x, (const float*)mix_all, mix_stride, first, count, (float*)out, d, vec);
     return NI_LAUNCH_RESULT();
 }

@@ -36,6 +36,11 @@ class Model:
                 raise ValueError(f"the order names block {run.block}, the model has {len(self.blocks)}")
             if run.enter is not None and self.pass_input is None:
                 raise ValueError(f"an entry of the order adds row {run.enter} of a pass input, the model has none")
+        # blocks over several streams a token hand the streams on among themselves: all of them or none
+        kinds = {getattr(self.blocks[run.block], "streams", None) for run in spec.order}
+        if len(kinds) > 1 or (kinds and kinds != {None} and (self.pass_input is not None or self.stream_mix is not None)):
+            raise ValueError("the blocks of a model over several streams all have the same number of them, "
+                             "and nothing else (a pass input, a mix of earlier states) works on the stream")
         self._needs: Dict[int, CacheNeed] = {}
         # an embedding that keeps something per request (the token before a portion's first) gets a cache of its
         # own behind the layers' and is handed it with every step
@@ -79,7 +84,7 @@ class Model:
 
     def _settled(self, h, pending):
         """A copy of the stream with what is pending added (for :attr:`tap`; the pass itself goes on as it was)."""
-        if hasattr(pending, "add_to"):          # a sum that was left to the block behind
+        if hasattr(pending, "add_to"):          # a sum that was left to the block behind (several streams: their sum)
             return pending.add_to(h.clone())
         pending = pending_for(None, pending, self.rt.dtype)
         return h.clone() if pending is None else h + pending.to(h.dtype)
@@ -144,7 +149,10 @@ class Model:
                 self.tap(i, h if pending is None else self._settled(h, pending))
         if ctx.logit_rows is None or ctx.logit_rows.shape[0] == 0:
             return None
-        x = self.final_norm.forward(h, pending_for(self.final_norm, pending, self.rt.dtype), rows=ctx.logit_rows)
+        if hasattr(pending, "normed"):          # streams that are summed and normed in one pass, for the wanted rows alone
+            x = pending.normed(h, self.final_norm, ctx.logit_rows, self.rt.dtype)
+        else:
+            x = self.final_norm.forward(h, pending_for(self.final_norm, pending, self.rt.dtype), rows=ctx.logit_rows)
         if logits_out is not None and getattr(self.head, "writes_into", False):
             return self.head.forward(x, out=logits_out[:x.shape[0]])
         return self.head.forward(x)

@@ -882,7 +882,8 @@ def skinny_gemm(x, weight, out: torch.Tensor, swiglu: bool = False, residual: bo
     """``x . weight^T`` for at most 64 rows of ``x``, streaming ``weight`` once (MFMA).  ``out``
     may be float32 for bfloat16 inputs.  With ``swiglu`` the weight is a stacked [2I, K] matrix
     (gate rows, then up rows) and ``out`` [M, I] receives ``silu(gate) * up`` (``activation`` "gelu_tanh": gelu in its
-    tanh form in silu's place, for a plain ``x``).  With ``residual``
+    tanh form in silu's place, for a plain ``x``); without it, ``activation`` "relu2" stores ``relu(x . weight^T)^2`` in the
+    input type.  With ``residual``
     ``out`` is the float32 residual stream [M, N] and the product is added into it, after the
     ``pending`` addends [S, M, N] that the stream has not received yet (at most 16 rows).  ``x`` may
     be a :class:`NormedInput` or a :class:`ScaledInput`.  With ``residual`` and ``leave`` (the norm that
@@ -918,7 +919,9 @@ def skinny_gemm(x, weight, out: torch.Tensor, swiglu: bool = False, residual: bo
         if not (out.dtype in (dtype, torch.float32)):
             raise KernelError(f"out must be {dtype} or float32")
         _gpu(out, "out", None, (M, N))
-        epi = 1 if (out.dtype == torch.float32 and dtype != torch.float32) else 0
+        if activation == "relu2" and (out.dtype != dtype or normed):
+            raise KernelError("relu2 is stored in the input type, for a given x")
+        epi = 5 if activation == "relu2" else 1 if (out.dtype == torch.float32 and dtype != torch.float32) else 0
     if pending is not None and not (residual and M <= SKINNY_BEST_ROWS):
         raise KernelError("pending addends go with the residual epilogue of at most 16 rows")
     if leave is not None and not residual:
@@ -1180,6 +1183,15 @@ def linear_swiglu(x, weight_gate_up, activation: str = "silu") -> torch.Tensor:
     return swiglu(torch.mm(x, rows_t), out, activation)
 
 
+def linear_relu2(x, weight) -> torch.Tensor:
+    """``relu(x . weight^T)^2`` in the type of ``x``: fused into the product for few rows, product then an elementwise kernel
+    for many."""
+    if skinny_wins(x.shape[0], x.shape[1], x.dtype, weight):
+        out = torch.empty(x.shape[0], weight.shape[0], dtype=x.dtype, device=x.device)
+        return skinny_gemm(x, weight, out, activation="relu2")
+    return experts_act(linear(x, weight), None, weight.shape[0], "relu2")
+
+
 def require_gpu() -> torch.device:
     if not torch.cuda.is_available():
         raise KernelError("no GPU is visible: nanoinfer_amd runs on an MI355X only and has no CPU path")
@@ -1194,7 +1206,7 @@ from .stream import (BIAS_ATTENTION_MFMA_FROM, DELTA_RUN_FROM, EXPERTS_FEW_ROWS,
                      bias_attention, bias_attention_lib, bias_attention_mfma, bias_attention_mfma_rows, bias_attention_rows, bias_attention_runs, delta_rule, delta_rule_lib, embed_scaled, experts_act, experts_few,
                      gated_side, kv_store, route_top, stream_add, stream_lib, embed_pair_hash, add_rows_vector, qk_norm_rope_store,
                      depth_mix, gate_heads, heads_apart, poly_norm, rmsnorm_cols, scale_, gate_rows, gather_pages, rows_to_pages,
-                     post_norm, merge_maps, EXPERT_FORMS, ROUTE_SCORINGS)
+                     post_norm, merge_maps, EXPERT_FORMS, ROUTE_SCORINGS, identity_experts, link_streams, LINK_STREAMS_MAX)
 # mixers with a state of fixed size: linear attention with a decay a head, the selective scan
 from .state import (conv_silu, decay_attention, decay_in_runs, decay_state_floats, gated_rmsnorm, scan_state_floats, selective_scan,  # noqa: E402,F401
                     silu_rows, state_mixers_lib, gated_memory, memory_norm, memory_state_floats)

@@ -33,8 +33,10 @@ _float = ctypes.c_float
 # ------------------------------------------------------------------ the residual stream
 
 def embed_scaled(ids: torch.Tensor, positions: torch.Tensor, table: torch.Tensor, pos_table: Optional[torch.Tensor],
-                 scale: float, out: torch.Tensor) -> torch.Tensor:
-    """``out[t] = table[ids[t]] * scale + pos_table[positions[t]]`` as float32 (no position rows: the first term)."""
+                 scale: float, out: torch.Tensor, freq: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[t] = table[ids[t]] * scale + pos_table[positions[t]]`` as float32 (no position rows: the first term).
+    ``freq`` float64 [(d + 1) // 2]: a sinusoid of the position is added, column 2i ``sin(position * freq[i])`` and column
+    2i + 1 the cosine."""
     T = ids.shape[0]
     vocab, d = table.shape
     _gpu(ids, "ids", torch.int32, (T,))
@@ -45,8 +47,10 @@ def embed_scaled(ids: torch.Tensor, positions: torch.Tensor, table: torch.Tensor
     if pos_table is not None:
         max_pos = pos_table.shape[0]
         _gpu(pos_table, "pos_table", table.dtype, (max_pos, d))
+    if freq is not None:
+        _gpu(freq, "freq", torch.float64, ((d + 1) // 2,))
     _check(stream_lib().ni_embed_scaled(_ptr(ids), _ptr(positions), _ptr(table), _ptr(pos_table), _ptr(out), T, d, vocab,
-                                        max_pos, _float(scale), dtype_code(table.dtype), _stream()), "embed_scaled")
+                                        max_pos, _float(scale), _ptr(freq), dtype_code(table.dtype), _stream()), "embed_scaled")
     return out
 
 
@@ -162,6 +166,55 @@ def post_norm(h: torch.Tensor, addends: Optional[torch.Tensor], alpha: float, we
     return h
 
 
+LINK_STREAMS_MAX = 32       # streams a token may have
+
+
+def link_streams(h: torch.Tensor, streams: int, addends: Optional[torch.Tensor], mix: Optional[torch.Tensor], out_w: Optional[torch.Tensor],
+                 in_w: Optional[torch.Tensor], norm_w: Optional[torch.Tensor], eps: float, v: torch.Tensor,
+                 h_out: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """What stands between two sublayers of a model whose tokens have several ``streams``, all float32:
+
+        ``x_t <- sum_f mix[f, t] x_f + out_w[t] * (sum of addends)``     (``mix`` None: no sublayer has run yet)
+        ``v = rmsnorm(sum_s in_w[s] x_s) * norm_w``                       (``in_w`` None: the plain sum; ``norm_w`` None: no norm)
+
+    ``h`` [T, streams, d], or [T, d] where a token's streams are all still equal; ``addends`` [T, d] or [n, T, d]; the new
+    streams go to ``h_out`` [T, streams, d] (``h`` itself, if it has that shape; None: nobody wants them); ``v`` [T, d] in a
+    compute type, or, with ``rows`` int32 [R], [R, d] for those rows alone."""
+    T, d = h.shape[0], h.shape[-1]
+    _gpu(h, "h", torch.float32)
+    _need(1 <= streams <= LINK_STREAMS_MAX, f"{streams} streams: 1 to {LINK_STREAMS_MAX} are compiled")
+    _need(h.dim() == 2 or tuple(h.shape) == (T, streams, d), f"h is {tuple(h.shape)}, not [T, d] or [T, {streams}, d]")
+    _need((mix is None) == (out_w is None), "the streams' mix and the sublayer's weights go together")
+    n = 0
+    if mix is not None:
+        _gpu(mix, "mix", torch.float32, (streams, streams))
+        _gpu(out_w, "out_w", torch.float32, (streams,))
+    if addends is not None:
+        _need(mix is not None, "a sublayer's output needs its mix")
+        _gpu(addends, "addends", torch.float32)
+        _need(addends.shape[-2:] == (T, d) and addends.dim() in (2, 3), "addends are float32 [T, d] or [n, T, d]")
+        n = 1 if addends.dim() == 2 else addends.shape[0]
+    if in_w is not None:
+        _gpu(in_w, "in_w", torch.float32, (streams,))
+    if norm_w is not None:
+        _gpu(norm_w, "norm_w", torch.float32, (d,))
+    R = T
+    if rows is not None:
+        R = rows.shape[0]
+        _gpu(rows, "rows", torch.int32, (R,))
+        _need(h_out is None, "new streams are written for all rows, not for some")
+    if h_out is not None:
+        _need(mix is not None, "streams that no sublayer has moved are not written again")
+        _gpu(h_out, "h_out", torch.float32, (T, streams, d))
+    _gpu(v, "v", None, (R, d))
+    err = stream_lib().ni_link_streams(_ptr(h), 1 if h.dim() == 2 else streams, _ptr(addends), n, _ptr(mix), _ptr(out_w), _ptr(in_w), _ptr(norm_w),
+                                       _float(eps), _ptr(h_out), _ptr(v), dtype_code(v.dtype), _ptr(rows), R, T, streams, d, _stream())
+    if err == -2:
+        raise KernelError(f"rows of {d} elements do not fit the kernel's memory")
+    _check(err, "link_streams")
+    return v
+
+
 def rmsnorm_cols(rows: torch.Tensor, col: int, weight: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
     """``x / sqrt(mean(x^2) + eps) * weight`` over the columns ``col .. col + len(weight)`` of ``rows`` float32 [T, wide]
     (some of a stacked product's accumulators); [T, len(weight)] in ``out_dtype``."""
@@ -275,15 +328,16 @@ def heads_apart(x: torch.Tensor, H: int, n: int) -> torch.Tensor:
 
 # ------------------------------------------------------------------ router and experts
 
-ROUTE_SCORINGS = {"softmax_chosen": 0, "softmax_all": 1, "sigmoid": 2}
+ROUTE_SCORINGS = {"softmax_chosen": 0, "softmax_all": 1, "sigmoid": 2, "softmax_share": 3}
 
 
 def route_top(z: torch.Tensor, top: int, mix_all: bool, over_all: bool = False, groups: int = 1, keep: int = 1,
               scoring: Optional[str] = None, correction: Optional[torch.Tensor] = None, group_top: int = 1, scale: float = 1.0):
     """The ``top`` experts of every row of ``z`` float32 [T, E] and their weights.  ``scoring``: "softmax_chosen" (an
     expert's value is its logit, the weights the softmax among the chosen; the default), "softmax_all" (``over_all``:
-    the softmax over all E experts, not renormalised) or "sigmoid" (the value is ``sigmoid(logit)``, the weights the
-    values themselves); every weight times ``scale``.  ``correction`` float32 [E] is added to the values that choose,
+    the softmax over all E experts, not renormalised), "sigmoid" (the value is ``sigmoid(logit)``, the weights the
+    values themselves) or "softmax_share" (the value is the softmax over all E experts, the weights the chosen values over
+    their sum + 1e-20); every weight times ``scale``.  ``correction`` float32 [E] is added to the values that choose,
     never to the weights.  With ``groups`` > 1 the experts form that many equal groups of neighbours, a group counts as
     much as the sum of its ``group_top`` largest choosing values, and only experts of the ``keep`` best groups can be
     chosen.  ``(chosen int32 [T, top], mix float32 [T, top], mix over all experts float32 [T, E] or None)``."""
@@ -322,19 +376,20 @@ def experts_act(up: torch.Tensor, mix_all: Optional[torch.Tensor], ff: int, gate
     """``mix_all[t, e] * relu(up[t, e * ff + i])^2`` in the type of ``up``; ``gated`` (True or "swiglu"): an expert's
     columns of ``up`` are [gate: ff | up: ff] and the result is ``mix_all[t, e] * silu(gate) * up``, [T, E * ff];
     "capped_glu": ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``, ``mix * g * sigmoid(slope * g) * (u + 1)``.
-    ``mix_all`` None (gated forms): every expert counts once."""
+    ``mix_all`` None: every expert counts once.  A row of ``mix_all`` may hold more numbers than there are experts; those
+    behind them are not looked at."""
     T, width = up.shape
     form = _expert_form(gated)
     _gpu(up, "up")
-    if mix_all is None:
-        _need(form != 0 and width % (2 * ff) == 0, "without a mix the rows are whole gated experts")
-        E = width // (2 * ff)
-    else:
-        E = mix_all.shape[1]
-        _gpu(mix_all, "mix_all", torch.float32, (T, E))
-    _need(width == E * ff * (2 if form else 1), "the experts' hidden rows do not match the router")
+    per = ff * (2 if form else 1)
+    _need(width % per == 0, "the rows are not whole experts")
+    E, stride = width // per, 0
+    if mix_all is not None:
+        stride = mix_all.shape[1]
+        _gpu(mix_all, "mix_all", torch.float32, (T, stride))
+        _need(stride >= E, "the experts' hidden rows do not match the router")
     act = torch.empty(T, E * ff, dtype=up.dtype, device=up.device)
-    _check(stream_lib().ni_experts_act(_ptr(up), _ptr(mix_all), _ptr(act), T, E, ff, form, _float(limit), _float(slope),
+    _check(stream_lib().ni_experts_act(_ptr(up), _ptr(mix_all), stride, _ptr(act), T, E, ff, form, _float(limit), _float(slope),
                                        dtype_code(up.dtype), _stream()), "experts_act")
     return act
 
@@ -346,7 +401,8 @@ def experts_few(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, chose
                 ff: int, gated=False, out: Optional[torch.Tensor] = None, limit: float = 0.0, slope: float = 1.0) -> torch.Tensor:
     """The weighted sum of the chosen experts for a few rows: ``w_up`` [E * ff, d] (``gated``: [E * 2 ff, d], an
     expert's gate rows and then its up rows; the hidden row is then ``silu(gate) * up`` instead of ``relu(up)^2``, or,
-    "capped_glu", the capped form of :func:`experts_act`), ``w_down`` [d, E * ff]; returns float32 [T, d] (``out``, if given)."""
+    "capped_glu", the capped form of :func:`experts_act`), ``w_down`` [d, E * ff]; a chosen index of E or more is an expert
+    whose output is its input; returns float32 [T, d] (``out``, if given)."""
     T, d = x.shape
     top = chosen.shape[1]
     form = _expert_form(gated)
@@ -365,6 +421,19 @@ def experts_few(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, chose
     _check(stream_lib().ni_experts_few(_ptr(x), _ptr(w_up), _ptr(w_down), _ptr(chosen), _ptr(mix), _ptr(hid), _ptr(out),
                                        T, d, ff, E, top, form, _float(limit), _float(slope), dtype_code(x.dtype), _stream()),
            "experts_few")
+    return out
+
+
+def identity_experts(x: torch.Tensor, mix_all: torch.Tensor, first: int, out: torch.Tensor) -> torch.Tensor:
+    """``out[t] = x[t] * (sum of mix_all[t, first:])``, float32 [T, d]: what the router outputs from ``first`` on add, whose
+    experts give their input back."""
+    T, d = x.shape
+    _gpu(x, "x")
+    _gpu(mix_all, "mix_all", torch.float32)
+    _need(mix_all.dim() == 2 and mix_all.shape[0] == T and 0 <= first < mix_all.shape[1], "no router outputs behind the experts")
+    _gpu(out, "out", torch.float32, (T, d))
+    _check(stream_lib().ni_identity_experts(_ptr(x), _ptr(mix_all), mix_all.shape[1], first, mix_all.shape[1] - first, _ptr(out), T, d,
+                                            dtype_code(x.dtype), _stream()), "identity_experts")
     return out
 
 

@@ -46,7 +46,9 @@ def _padded_cols(w: torch.Tensor, cols: int) -> torch.Tensor:
 class ScaledTableEmbedding(Part):
     """``h[t] = E[id[t]] * scale + P[position[t]]``; the position rows are learned and not scaled.  With a ``norm``
     among the weights the row is then divided by its root mean square and multiplied by that weight, in float32.
-    params: vocab_size, hidden_size, scale, max_positions, eps (of the norm).  weights: weight [vocab, hidden], positions
+    With ``sinusoid_base`` b a vector of the position p is added: column 2i ``sin(p * b^(-2i / hidden))``, column 2i + 1 the
+    cosine of the same angle, the angle in float64.
+    params: vocab_size, hidden_size, scale, max_positions, eps (of the norm), sinusoid_base (absent: none).  weights: weight [vocab, hidden], positions
     [max_positions, hidden] (absent from the spec's weights: no position rows), norm [hidden] (absent: no norm)."""
 
     graph_safe = True
@@ -69,10 +71,14 @@ class ScaledTableEmbedding(Part):
         self.positions = rt.matrix(spec.weights["positions"], weights["positions"]) if "positions" in spec.weights else None
         self.norm = rt.vector32(spec.weights["norm"], weights["norm"]) if "norm" in spec.weights else None
         self.eps = float(spec.params.get("eps", 0.0))
+        self.freq = None
+        if spec.params.get("sinusoid_base") is not None:
+            d, base = self.hidden_size, float(spec.params["sinusoid_base"])
+            self.freq = torch.tensor([base ** (-2.0 * i / d) for i in range((d + 1) // 2)], dtype=torch.float64).to(rt.device)
 
     def forward(self, token_ids: torch.Tensor, ctx=None) -> torch.Tensor:
         out = torch.empty(token_ids.shape[0], self.hidden_size, dtype=torch.float32, device=self.rt.device)
-        K.embed_scaled(token_ids, ctx.positions, self.weight, self.positions, self.scale, out)
+        K.embed_scaled(token_ids, ctx.positions, self.weight, self.positions, self.scale, out, freq=self.freq)
         return out if self.norm is None else K.post_norm(out, None, 1.0, self.norm, self.eps)
 
 
@@ -400,19 +406,22 @@ class RoutedExperts(Part):
     "capped_glu" (``g = min(W_gate x, limit)``, ``u = clamp(W_up x, -limit, limit)``, ``W_down (g sigmoid(slope g) (u + 1))``,
     with the params ``limit`` and ``slope``);
     mix: "softmax_chosen" (the softmax over the chosen logits alone, the default), "softmax_all" (the softmax over all
-    experts, the chosen ones' shares not renormalised) or "sigmoid" (an expert's score is the sigmoid of its logit, and the
-    chosen ones' scores are their weights as they are); mix_scale (default 1) multiplies every weight;
+    experts, the chosen ones' shares not renormalised), "sigmoid" (an expert's score is the sigmoid of its logit, and the
+    chosen ones' scores are their weights as they are) or "softmax_share" (an expert's score is its share of the softmax over
+    all, which a correction is added to, and the chosen ones' weights are their scores over their sum); mix_scale (default 1) multiplies every weight;
     groups, keep (default 1, 1): the experts form ``groups`` equal groups of neighbours, a group counts as much as the
     sum of its ``group_top`` (default 1) best experts, and only the best ``keep`` groups can be chosen from;
+    identity (default 0): the router has that many outputs behind the experts', whose experts have no tensors: their output is
+    the input x itself;
     shared: None or the PartSpec of a feed-forward.
-    weights: router [experts, d], up<e> [expert_size, d], down<e> [d, expert_size], with a gated activation also gate<e>;
-    correction [experts] (absent: none): added to the scores that choose the experts and the groups, never to the weights.
+    weights: router [experts + identity, d], up<e> [expert_size, d], down<e> [d, expert_size], with a gated activation also gate<e>;
+    correction [experts + identity] (absent: none): added to the scores that choose the experts and the groups, never to the weights.
 
     The experts' matrices are laid side by side, up [E * ff, d] (gated: [E * 2 ff, d], an expert's gate rows and then
     its up rows) and down [d, E * ff].  For a few rows only the chosen experts' rows are read; for many, all experts
     run as two dense products with the mix of an expert that was not chosen at zero, which the matrix cores do
-    faster than a gather would here.  With a shared expert the result is two float32 addends [2, T, d], which the
-    next norm sums in float32."""
+    faster than a gather would here.  With a shared expert, and in steps of many rows with identity experts, the result is
+    two or three float32 addends [n, T, d], which the next norm sums in float32."""
 
     graph_safe = True
 
@@ -420,9 +429,10 @@ class RoutedExperts(Part):
     def weight_requests(cls, spec):
         p, w = spec.params, spec.weights
         d, ff = p["hidden_size"], p["expert_size"]
-        out = [WeightRequest(w["router"], (p["experts"], d))]
+        outputs = p["experts"] + p.get("identity", 0)
+        out = [WeightRequest(w["router"], (outputs, d))]
         if "correction" in w:
-            out.append(WeightRequest(w["correction"], (p["experts"],)))
+            out.append(WeightRequest(w["correction"], (outputs,)))
         for e in range(p["experts"]):
             if p.get("activation", "relu2") != "relu2":
                 out.append(WeightRequest(w[f"gate{e}"], (ff, d)))
@@ -435,7 +445,8 @@ class RoutedExperts(Part):
     def __init__(self, spec, weights, rt):
         super().__init__(spec, weights, rt)
         p, names = spec.params, spec.weights
-        self.E, self.top, self.ff = int(p["experts"]), int(p["top"]), int(p["expert_size"])
+        self.E, self.top, self.ff, self.identity = int(p["experts"]), int(p["top"]), int(p["expert_size"]), int(p.get("identity", 0))
+        outputs = self.E + self.identity        # of the router
         activation = p.get("activation", "relu2")
         if activation not in K.EXPERT_FORMS:
             raise ValueError(f"expert activation {activation!r} is not known (known: {sorted(K.EXPERT_FORMS)})")
@@ -450,8 +461,8 @@ class RoutedExperts(Part):
         self.mix_scale = float(p.get("mix_scale", 1.0))
         self.groups, self.keep, self.group_top = int(p.get("groups", 1)), int(p.get("keep", 1)), int(p.get("group_top", 1))
         self.correction = rt.vector32(names["correction"], weights["correction"]) if "correction" in names else None
-        if self.groups < 1 or self.E % self.groups or not 1 <= self.keep <= self.groups or self.top > self.E // self.groups * self.keep:
-            raise ValueError(f"{self.top} experts cannot be chosen from {self.keep} of {self.groups} groups of {self.E}")
+        if self.groups < 1 or outputs % self.groups or not 1 <= self.keep <= self.groups or self.top > outputs // self.groups * self.keep:
+            raise ValueError(f"{self.top} experts cannot be chosen from {self.keep} of {self.groups} groups of {outputs}")
         self.w_router = rt.weight(names["router"], weights["router"])
         order = [k for e in range(self.E) for k in ((f"gate{e}", f"up{e}") if self.gated else (f"up{e}",))]
         self.w_up = rt.weight("|".join(names[k] for k in order), torch.cat([weights[k] for k in order], dim=0), tiled=False)
@@ -467,18 +478,23 @@ class RoutedExperts(Part):
         few = T <= K.EXPERTS_FEW_ROWS
         chosen, mix, mix_all = K.route_top(z, self.top, mix_all=not few, groups=self.groups, keep=self.keep, scoring=self.mix,
                                            correction=self.correction, group_top=self.group_top, scale=self.mix_scale)
+        # addends beside the routed experts' own sum: the shared expert's, and in the dense way the identity experts'
+        more = int(self.shared is not None) + int(self.identity > 0 and not few)
         out = None
-        if self.shared is not None:
-            out = torch.empty(2, T, self.w_down.shape[0], dtype=torch.float32, device=x.device)
+        if more:
+            out = torch.empty(1 + more, T, self.w_down.shape[0], dtype=torch.float32, device=x.device)
         if few:
             y = K.experts_few(x, self.w_up.rows, self.w_down.rows, chosen, mix, self.ff, self.activation, None if out is None else out[0],
                               limit=self.limit, slope=self.slope)
         else:
             act = K.experts_act(K.linear(x, self.w_up), mix_all, self.ff, self.activation, self.limit, self.slope)
             y = K.linear(act, self.w_down, out_dtype=torch.float32, out=None if out is None else out[0])
+            if self.identity:
+                K.identity_experts(x, mix_all, self.E, out[more])
         if out is None:
             return y
-        K.linear(self.shared.hidden(x), self.shared.w_down, out_dtype=torch.float32, out=out[1])
+        if self.shared is not None:
+            K.linear(self.shared.hidden(x), self.shared.w_down, out_dtype=torch.float32, out=out[1])
         return out
 
 

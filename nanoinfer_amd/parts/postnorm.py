@@ -36,7 +36,9 @@ class SinkAttention(WindowAttention):
     earlier key).  In float32: an RMS norm of every query head and of every key head on its own, each with one weight
     shared by the heads; then the rotation of the first channels of every head (``position``; ``adjacent_pairs``: channel
     2i turns with channel 2i + 1); ``score = q . k * scale``; the softmax's denominator holds one more term
-    ``exp(sink[h])`` that has no key and no value; head h's output is multiplied by ``sigmoid(W_g x)[h]``; then ``W_o``.
+    ``exp(sink[h])`` that has no key and no value; head h's output is multiplied by ``sigmoid(W_g x)[h]``, or, with ``gate``
+    "channel", every channel of every head by a gate of its own; then ``W_o``.  A query at position p may be multiplied by
+    ``1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)`` (``temp_coef`` None: not); ``position`` None: no rotation.
 
     A part with ``shares_kv`` has no key and value projections: it reads the keys (normed and rotated) and values that
     another entry of the order wrote (``LayerRun.writes_cache`` False) with its own queries, window, sink and gate.
@@ -44,8 +46,8 @@ class SinkAttention(WindowAttention):
     every key).
 
     params: hidden_size, num_heads, num_kv_heads, key_dim, value_dim, scale, window, cache_window, eps, position,
-    adjacent_pairs, shares_kv.
-    weights: q [H*dk, d], q_norm [dk], sink [H], g [H, d], o [d, H*dv]; without ``shares_kv`` also k [G*dk, d],
+    adjacent_pairs, shares_kv, gate ("head", the default, or "channel"), temp_coef, temp_every.
+    weights: q [H*dk, d], q_norm [dk], sink [H], g [H, d] (a gate a channel: [H*dv, d]), o [d, H*dv]; without ``shares_kv`` also k [G*dk, d],
     v [G*dv, d], k_norm [dk]."""
 
     graph_safe = True
@@ -54,8 +56,9 @@ class SinkAttention(WindowAttention):
     def weight_requests(cls, spec):
         p, w = spec.params, spec.weights
         d, H, G, dk, dv = p["hidden_size"], p["num_heads"], p["num_kv_heads"], p["key_dim"], p["value_dim"]
+        gates = H * dv if p.get("gate", "head") == "channel" else H
         out = [WeightRequest(w["q"], (H * dk, d)), WeightRequest(w["q_norm"], (dk,)), WeightRequest(w["sink"], (H,)),
-               WeightRequest(w["g"], (H, d)), WeightRequest(w["o"], (d, H * dv))]
+               WeightRequest(w["g"], (gates, d)), WeightRequest(w["o"], (d, H * dv))]
         if not p.get("shares_kv"):
             out += [WeightRequest(w["k"], (G * dk, d)), WeightRequest(w["v"], (G * dv, d)), WeightRequest(w["k_norm"], (dk,))]
         if p.get("position") is not None:
@@ -76,6 +79,10 @@ class SinkAttention(WindowAttention):
         self.head_q_norm = rt.vector32(names["q_norm"], weights["q_norm"])
         self.head_k_norm = None if self.shares_kv else rt.vector32(names["k_norm"], weights["k_norm"])
         self.core.sink = rt.vector32(names["sink"], weights["sink"])
+        gate = p.get("gate", "head")
+        if gate not in ("head", "channel"):
+            raise ValueError(f"gate {gate!r} is not 'head' or 'channel'")
+        self.gate_every = self.dv if gate == "head" else 1
         self.gate_col = self.H * self.dk + (0 if self.shares_kv else self.G * (self.dk + self.dv))
 
     def _stacked_projection(self, names, weights, rt):
@@ -98,7 +105,7 @@ class SinkAttention(WindowAttention):
             K.qk_norm_rope_store(proj, ctx.positions, cache.slot_mapping, self.head_q_norm, self.head_k_norm, self.eps, self.freq,
                                  self.amplitude, q, cache.kpool, cache.vpool, self.H, per_head=True, adjacent=self.adjacent)
         attended = self.attend(q, ctx, cache, self.window, 0, 1.0)
-        gated = K.gate_rows(attended, proj, self.gate_col, out=attended, every=self.dv)
+        gated = K.gate_rows(attended, proj, self.gate_col, out=attended, every=self.gate_every)
         return K.linear(gated, self.w_o, out_dtype=torch.float32, out=out)
 
 
