@@ -495,6 +495,27 @@ def fanidra_config(layers: int, vocab: int, like: dict) -> dict:
             "layers": [dict(memory if i % 2 == 0 else attn, mlp={"ff": ff, "kind": "dense"}) for i in range(layers)]}
 
 
+def fuvevik_config(layers: int, vocab: int, like: dict) -> dict:
+    """A Fuvevik model whose layers have the sizes of a Llama shape's over four streams a token: attention over every key
+    (the shape's heads and head size, a query factor), every fourth layer on the keys and values of the one before; dense
+    feed-forwards of the shape's size and the routed experts of the Vimilix shape (sixteen of an eighth of it, beside two
+    that give their input back, of which a token uses four, and a shared expert of a quarter of it, capped), in turn."""
+    width, ff, hd = like["hidden_size"], like["intermediate_size"], like["head_dim"]
+    attn = {"heads": like["num_attention_heads"], "kv_heads": like["num_key_value_heads"], "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+            "q_temp": {"coef": 0.1, "every": 1024}}
+    dense = {"kind": "dense", "ff": ff}
+    routed = {"kind": "moe", "expert": {"ff": ff // 8, "limit": 7.0}, "router": {"experts": 16, "identity": 2, "top": 4},
+              "shared": {"ff": ff // 4, "limit": 7.0}}
+    return {"architecture": "Fuvevik", "vocab": vocab, "width": width, "streams": 4, "norm": {"eps": 1e-5},
+            "layers": [{"type": "attention", "mixer": dict(attn, kv_from=i - 1) if i % 4 == 3 else attn, "mlp": routed if i % 2 else dense}
+                       for i in range(layers)]}
+
+
+# workload -> the model it is about, the framework's closest other model beside it
+PAIRS = {"hybrid": ("zekalorn", "llama"), "stateful": ("fusavik", "zekalorn"), "latent": ("ruludra", "fusavik"),
+         "postnorm": ("vimilix", "fusavik"), "differential": ("fanidra", "ruludra"), "streams": ("fuvevik", "vimilix")}
+
+
 def hybrid(args) -> int:
     """``--workload hybrid``: prefill of one prompt and decode steps of the Zekalorn shape above and of the Llama
     shape of equal depth, one JSON line with both.  ``--workload stateful``: the same of the Fusavik shape above
@@ -504,27 +525,25 @@ def hybrid(args) -> int:
     the Vimilix shape above beside the Fusavik shape (the framework's other model with attention in a window and routed
     experts chosen within groups beside a shared one).  ``--workload differential``: the same of the Fanidra shape above
     beside the Ruludra shape (the framework's other model with a gated memory a head, attention in a window, normed
-    sublayer outputs and dense feed-forwards)."""
+    sublayer outputs and dense feed-forwards).  ``--workload streams``: the same of the Fuvevik shape above beside the
+    Vimilix shape (the framework's other model with a sink and a gate in its attention, keys and values that later layers
+    read again, and capped routed experts beside a shared one)."""
     import torch
     torch.cuda.set_device(0)
     layers = args.layers or 8
     prompt, batch = args.prompt_len, args.batch
-    first = {"stateful": "fusavik", "latent": "ruludra", "postnorm": "vimilix", "differential": "fanidra"}.get(args.workload, "zekalorn")
+    first = PAIRS[args.workload][0]
     out = {"metric": f"{args.workload}_decode_tokens_per_s", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
            "higher_is_better": True, "dtype": args.dtype, "data": "synthetic token ids, random-init weights",
            "config": {"layers": layers, "prompt_len": prompt, "global_batch": batch, "shape": args.shape,
                       "width": SHAPES[args.shape][2]["hidden_size"], "vocab": 128256}}
     like = SHAPES[args.shape][2]
-    shapes = {"zekalorn": hybrid_config(layers, 128256, prompt + 2048, like),
-              "llama": dict(like, num_hidden_layers=layers, max_position_embeddings=prompt + 2048)}
-    if args.workload == "stateful":
-        shapes = {"fusavik": fusavik_config(layers, 128256, like), "zekalorn": shapes["zekalorn"]}
-    if args.workload == "latent":
-        shapes = {"ruludra": ruludra_config(layers, 128256, like), "fusavik": fusavik_config(layers, 128256, like)}
-    if args.workload == "postnorm":
-        shapes = {"vimilix": vimilix_config(layers, 128256, like), "fusavik": fusavik_config(layers, 128256, like)}
-    if args.workload == "differential":
-        shapes = {"fanidra": fanidra_config(layers, 128256, like), "ruludra": ruludra_config(layers, 128256, like)}
+    makers = {"zekalorn": lambda: hybrid_config(layers, 128256, prompt + 2048, like),
+              "llama": lambda: dict(like, num_hidden_layers=layers, max_position_embeddings=prompt + 2048),
+              "fusavik": lambda: fusavik_config(layers, 128256, like), "ruludra": lambda: ruludra_config(layers, 128256, like),
+              "vimilix": lambda: vimilix_config(layers, 128256, like), "fanidra": lambda: fanidra_config(layers, 128256, like),
+              "fuvevik": lambda: fuvevik_config(layers, 128256, like)}
+    shapes = {name: makers[name]() for name in PAIRS[args.workload]}
     for name, cfg in shapes.items():
         if args.only and name != args.only:
             continue
@@ -581,16 +600,17 @@ def main() -> int:
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64 and the further points")
     ap.add_argument("--no-further", action="store_true",
                     help="skip the points beyond the default line's: contexts of 8k and 32k, float32, the 3B shape")
-    ap.add_argument("--only", default=None, choices=["zekalorn", "llama", "fusavik", "ruludra", "vimilix", "fanidra"],
-                    help="hybrid, stateful, latent, postnorm, differential: measure one of the two models")
-    ap.add_argument("--workload", default="steps", choices=["steps", "serving", "hybrid", "stateful", "latent", "postnorm", "differential"],
+    ap.add_argument("--only", default=None, choices=sorted({name for pair in PAIRS.values() for name in pair}),
+                    help="hybrid, stateful, latent, postnorm, differential, streams: measure one of the two models")
+    ap.add_argument("--workload", default="steps", choices=["steps", "serving"] + list(PAIRS),
                     help="steps: the decode step and prefill of the result line's contract (default); "
                          "serving: concurrent requests through the engine's scheduler, a line of its own; "
                          "hybrid: prefill and decode of a Zekalorn model at the 1B shape's layer sizes beside the Llama shape; "
                          "stateful: the same of a Fusavik model beside the Zekalorn one; "
                          "latent: the same of a Ruludra model beside the Fusavik one; "
                          "postnorm: the same of a Vimilix model beside the Fusavik one; "
-                         "differential: the same of a Fanidra model beside the Ruludra one")
+                         "differential: the same of a Fanidra model beside the Ruludra one; "
+                         "streams: the same of a Fuvevik model beside the Vimilix one")
     ap.add_argument("--requests", type=int, default=64, help="serving: concurrent requests")
     ap.add_argument("--new-tokens", type=int, default=256, help="serving: tokens generated per request")
     ap.add_argument("--min-prompt", type=int, default=128, help="serving: shortest prompt")
@@ -611,7 +631,7 @@ def main() -> int:
         return 2
     if args.workload == "serving":
         return serving(args)
-    if args.workload in ("hybrid", "stateful", "latent", "postnorm", "differential"):
+    if args.workload in PAIRS:
         return hybrid(args)
     args.prefill_chunk = args.prefill_chunk or PREFILL_CHUNK
 
