@@ -22,6 +22,9 @@
 // over that map's keys and the kv head's values: H counts the query heads of all maps, G the (kv head, map) pairs.  What
 // becomes of the maps' outputs is up to `merge_maps`, which takes them as the kernels leave unfinished rows.
 //
+// A gate (`Gate`): an output channel c of head h is multiplied by sigmoid(g[token, (h * dv + c) / every]) when its row is
+// finished, the pre-activations g float32 rows (some columns of the projections the queries came from).
+//
 // A sink (`sink`, float32 [heads], or null) is one more term exp(sink[head]) in a row's denominator, with no key and
 // no value: the weights of a row then sum to less than one.  It counts once a row, whatever the number of runs: the
 // kernels add it when a row is finished (a row in runs: when the runs are merged).
@@ -133,11 +136,15 @@ qk_norm_rope_store_kernel(const float* __restrict__ proj, int row_stride, const 
     const float* row = proj + static_cast<size_t>(t) * row_stride;
     const int H = f.H, G = f.G, dq = f.dq, dk = f.dk, dv = f.dv, rot = f.rot;
     const int nq = H * dq, nk = G * dk;
+    const int slices = gridDim.y, slice = blockIdx.y;
+    const int per = ((nq + nk + slices - 1) / slices + 3) / 4 * 4;
     float rq = 1.f, rk = 1.f;
     if (f.per_head) {
-        // a head a wavefront at a time: its lanes walk the head's normed channels
+        // a head a wavefront at a time: its lanes walk the head's normed channels; only heads of this workgroup's share
         const int lane = tid & (WAVE - 1), wave = tid / WAVE, waves = blockDim.x / WAVE;
-        for (int hd = wave; hd < H + G; hd += waves) {
+        auto head_of = [&](int i) { return i < nq ? i / dq : H + (i - nq) / dk; };
+        const int i0 = slice * per, i1 = min(nq + nk, (slice + 1) * per);
+        for (int hd = i0 < i1 ? head_of(i0) + wave : H + G; hd <= (i0 < i1 ? head_of(i1 - 1) : -1); hd += waves) {
             const bool is_q = hd < H;
             const float* w = is_q ? wq : wk;
             if (!w) continue;                                  // the same for the whole wavefront
@@ -174,8 +181,6 @@ qk_norm_rope_store_kernel(const float* __restrict__ proj, int row_stride, const 
     }
     const int slot = slot_mapping ? slot_mapping[t] : -1;
     const int page = slot >= 0 ? slot / page_size : 0, in_page = slot >= 0 ? slot % page_size : 0;
-    const int slices = gridDim.y, slice = blockIdx.y;
-    const int per = ((nq + nk + slices - 1) / slices + 3) / 4 * 4;
     for (int i = slice * per + tid; i < min(nq + nk, (slice + 1) * per); i += blockDim.x) {
         const bool is_q = i < nq;
         const int j = is_q ? i : i - nq;                 // index inside the projection
@@ -365,6 +370,16 @@ __device__ __forceinline__ void stage_tile(const T* __restrict__ kpool, const T*
     stage_rows<T>(vpool, Vs, dvp, dv, dv, table, page_size, G, g, k0, k_last, v_pieces);
 }
 
+// The gate on an attention's output: see the top of the file (null rows: none)
+struct Gate {
+    const float* rows;
+    int stride, every;
+    // the factor on channel c of the H * dv of token t
+    __device__ __forceinline__ float of(size_t t, int c) const {
+        return rows ? 1.0f / (1.0f + expf(-rows[t * stride + (every == 1 ? c : c / every)])) : 1.f;
+    }
+};
+
 // What an attention may do beside the bias: see the top of the file (0, 0, 1: nothing)
 struct ScoreForm {
     float softcap;
@@ -378,7 +393,7 @@ bias_attention_kernel(const T* __restrict__ qkv, int row_stride, const T* __rest
                       const int32_t* __restrict__ positions, const float* __restrict__ bias, int distances, T* __restrict__ out, int H, int G, int dk, int dv,
                       int page_size, float scale, float temp_coef, int temp_every, int heads_per_chunk, int n_runs,
                       float* __restrict__ partial, bool k_pieces, bool v_pieces, int dkp, int window, int keep_first,
-                      float out_scale, const float* __restrict__ sink, ScoreForm form) {
+                      float out_scale, const float* __restrict__ sink, ScoreForm form, Gate gate) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     // a lane reads its key's row: the stride is the row plus four floats where rows are whole 16-byte pieces (read
     // as such), plus one otherwise; both spread the lanes over the banks
@@ -528,7 +543,7 @@ bias_attention_kernel(const T* __restrict__ qkv, int row_stride, const T* __rest
 #pragma unroll
         for (int cc = 0; cc < MAX_VCHUNKS; ++cc) {
             const int c = lane + cc * WAVE;
-            if (c < dv) st(orow + c, acc[rr][cc] * inv);
+            if (c < dv) st(orow + c, acc[rr][cc] * inv * gate.of(first_row + r / heads_here, head[rr] * dv + c));
         }
     }
 }
@@ -575,7 +590,7 @@ bias_attention_mfma_kernel(const T* __restrict__ qkv, int row_stride, const T* _
                            const int32_t* __restrict__ positions, const float* __restrict__ bias, int distances,
                            T* __restrict__ out, int H, int G, int dk, int dv, int page_size, float scale, float temp_coef,
                            int temp_every, int heads_per_chunk, bool k_pieces, bool v_pieces, int window, int keep_first,
-                           float out_scale, const float* __restrict__ sink, ScoreForm form, float* __restrict__ partial) {
+                           float out_scale, const float* __restrict__ sink, ScoreForm form, float* __restrict__ partial, Gate gate) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int dkp = dk + 4, dvp = dv + 4;         // strides that spread the sixteen rows of a read over the banks
     // keys and values that are one pool (dv = dk) are staged once: the values are read from the keys' tile
@@ -721,7 +736,8 @@ bias_attention_mfma_kernel(const T* __restrict__ qkv, int row_stride, const T* _
     for (int db = 0; db < DVB; ++db) {
         if (db < dvb) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) st(orow + 16 * db + r, acc[db][r] * inv);
+            for (int r = 0; r < 4; ++r)
+                st(orow + 16 * db + r, acc[db][r] * inv * gate.of(first_row + row / heads_here, head * dv + 16 * db + 4 * kg + r));
         }
     }
 }
@@ -762,7 +778,7 @@ bias_attention_bf16_kernel(const bf16_t* __restrict__ qkv, int row_stride, const
                            const int32_t* __restrict__ positions, const float* __restrict__ bias, int distances, bf16_t* __restrict__ out,
                            int H, int G, int dk, int dv, int page_size, float scale, float temp_coef, int temp_every, int heads_per_chunk,
                            int window, int keep_first, float out_scale, const float* __restrict__ sink, ScoreForm form,
-                           float* __restrict__ partial) {
+                           float* __restrict__ partial, Gate gate) {
     constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
     constexpr int KROW = 32 * KQ + TILE_PAD, VROW = 16 * DVB + TILE_PAD, VP = DVB / 2;
     __shared__ __attribute__((aligned(16))) uint16_t Ks[KEYS * KROW];
@@ -943,7 +959,11 @@ bias_attention_bf16_kernel(const bf16_t* __restrict__ qkv, int row_stride, const
 #pragma unroll
     for (int db = 0; db < DVB; ++db) {
         if (db < dvb) {
-            const float o[4] = {acc[db][0] * inv, acc[db][1] * inv, acc[db][2] * inv, acc[db][3] * inv};
+            float o[4] = {acc[db][0] * inv, acc[db][1] * inv, acc[db][2] * inv, acc[db][3] * inv};
+            if (gate.rows) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[r] *= gate.of(first_row + token, head * dv + 16 * db + 4 * kg + r);
+            }
             store_packed<bf16_t, 4>(orow + 16 * db, o);
         }
     }
@@ -956,7 +976,7 @@ bias_attention_bf16_kernel(const bf16_t* __restrict__ qkv, int row_stride, const
 // the runs' weights out for itself (lane r takes run r's maximum and sum, n_runs <= 64) and sums its own channels.
 template <typename T>
 __global__ void __launch_bounds__(MAX_VCHUNKS * WAVE) merge_runs_kernel(const float* __restrict__ partial, T* __restrict__ out, int n_runs,
-                                                                        int dv, float out_scale, const float* __restrict__ sink, int H) {
+                                                                        int dv, float out_scale, const float* __restrict__ sink, int H, Gate gate) {
     __shared__ float weight[MAX_VCHUNKS][WAVE];
     const size_t row = blockIdx.x;
     const float* p = partial + row * n_runs * (dv + 2);
@@ -980,7 +1000,7 @@ __global__ void __launch_bounds__(MAX_VCHUNKS * WAVE) merge_runs_kernel(const fl
             const float wr = weight[wave][r];
             if (wr > 0.f) a += p[r * (dv + 2) + 2 + c] * wr;
         }
-        st(out + row * dv + c, a * out_scale / L);
+        st(out + row * dv + c, a * out_scale / L * gate.of(row / H, static_cast<int>(row % H) * dv + c));
     }
 }
 
@@ -1104,12 +1124,14 @@ NI_EXPORT int ni_bias_attention(const void* qkv, int row_stride, const void* kpo
                                 int table_width, const void* tiles, int n_tiles, const void* positions, const void* bias, int distances, void* out,
                                 int H, int G, int dk, int dv, int page_size, float scale, float temp_coef, int temp_every,
                                 int heads_per_chunk, int n_runs, void* partial, int n_rows, int waves, int window, int keep_first,
-                                float out_scale, const void* sink, float softcap, int chunk, int maps, int unfinished, int dtype,
-                                hipStream_t stream) {
+                                float out_scale, const void* sink, float softcap, int chunk, int maps, int unfinished, const void* gate_rows,
+                                int gate_stride, int gate_every, int dtype, hipStream_t stream) {
     // `unfinished`: the rows stay in `partial`, runs unmerged (also a single run), for a kernel that finishes them; no sink
     if (n_tiles <= 0) return 0;
     if (window < 0 || keep_first < 0 || chunk < 0 || (chunk && window) || maps < 1 || G % maps) return -1;
-    if (unfinished && (!partial || sink)) return -1;
+    if (unfinished && (!partial || sink || gate_rows)) return -1;
+    if (gate_rows && (gate_every < 1 || gate_stride < (H * dv + gate_every - 1) / gate_every || maps != 1)) return -1;
+    const Gate gate{(const float*)gate_rows, gate_stride, gate_every};
     const ScoreForm form{softcap, chunk, maps};
     if (dv > MAX_VCHUNKS * WAVE || H % G || heads_per_chunk < 1 || heads_per_chunk > ROWS) return -1;
     const int group = H / G;
@@ -1133,9 +1155,9 @@ NI_EXPORT int ni_bias_attention(const void* qkv, int row_stride, const void* kpo
             (const float*)qkv, row_stride, (const float*)kpool, (const float*)vpool, (const int32_t*)block_table, table_width,
             (const int32_t*)tiles, (const int32_t*)positions, (const float*)bias, distances, (float*)out, H, G, dk, dv, page_size, scale, temp_coef,
             temp_every, heads_per_chunk, n_runs, (float*)partial, k_pieces, v_pieces, dkp, window, keep_first, out_scale,
-            (const float*)sink, form);
+            (const float*)sink, form, gate);
         if (partial && !unfinished) merge_runs_kernel<float><<<n_rows * H, std::min(MAX_VCHUNKS, (dv + WAVE - 1) / WAVE) * WAVE, 0, stream>>>((const float*)partial, (float*)out, n_runs, dv, out_scale,
-                                                                             (const float*)sink, H);
+                                                                             (const float*)sink, H, gate);
     } else {
         static size_t allowed = 48 * 1024;
         if (lds > allowed && (allowed = lds))
@@ -1145,9 +1167,9 @@ NI_EXPORT int ni_bias_attention(const void* qkv, int row_stride, const void* kpo
             (const bf16_t*)qkv, row_stride, (const bf16_t*)kpool, (const bf16_t*)vpool, (const int32_t*)block_table, table_width,
             (const int32_t*)tiles, (const int32_t*)positions, (const float*)bias, distances, (bf16_t*)out, H, G, dk, dv, page_size, scale, temp_coef,
             temp_every, heads_per_chunk, n_runs, (float*)partial, k_pieces, v_pieces, dkp, window, keep_first, out_scale,
-            (const float*)sink, form);
+            (const float*)sink, form, gate);
         if (partial && !unfinished) merge_runs_kernel<bf16_t><<<n_rows * H, std::min(MAX_VCHUNKS, (dv + WAVE - 1) / WAVE) * WAVE, 0, stream>>>((const float*)partial, (bf16_t*)out, n_runs, dv, out_scale,
-                                                                              (const float*)sink, H);
+                                                                              (const float*)sink, H, gate);
     }
     return NI_LAUNCH_RESULT();
 }
@@ -1167,7 +1189,7 @@ NI_EXPORT int ni_bias_attention_mfma_rows(int dk, int dv, int one_pool) {
 struct MfmaArgs {
     const void *qkv; int row_stride; const void *kpool, *vpool, *block_table; int table_width; const void *tiles, *positions, *bias;
     int distances; void* out; int H, G, dk, dv, page_size; float scale, temp_coef; int temp_every, heads_per_chunk;
-    bool k_pieces, v_pieces; int window, keep_first; float out_scale; const void* sink; ScoreForm form; void* partial;
+    bool k_pieces, v_pieces; int window, keep_first; float out_scale; const void* sink; ScoreForm form; void* partial; Gate gate;
 };
 
 template <typename T, int QS, int DVB>
@@ -1183,7 +1205,7 @@ static hipError_t launch_mfma(const MfmaArgs& a, dim3 grid, size_t lds, hipStrea
         (const T*)a.qkv, a.row_stride, (const T*)a.kpool, (const T*)a.vpool, (const int32_t*)a.block_table, a.table_width,
         (const int32_t*)a.tiles, (const int32_t*)a.positions, (const float*)a.bias, a.distances, (T*)a.out, a.H, a.G, a.dk, a.dv,
         a.page_size, a.scale, a.temp_coef, a.temp_every, a.heads_per_chunk, a.k_pieces, a.v_pieces, a.window, a.keep_first,
-        a.out_scale, (const float*)a.sink, a.form, (float*)a.partial);
+        a.out_scale, (const float*)a.sink, a.form, (float*)a.partial, a.gate);
     return hipSuccess;
 }
 
@@ -1193,7 +1215,7 @@ static void launch_bf16(const MfmaArgs& a, dim3 grid, hipStream_t stream) {
         (const bf16_t*)a.qkv, a.row_stride, (const bf16_t*)a.kpool, (const bf16_t*)a.vpool, (const int32_t*)a.block_table, a.table_width,
         (const int32_t*)a.tiles, (const int32_t*)a.positions, (const float*)a.bias, a.distances, (bf16_t*)a.out, a.H, a.G, a.dk, a.dv,
         a.page_size, a.scale, a.temp_coef, a.temp_every, a.heads_per_chunk, a.window, a.keep_first, a.out_scale, (const float*)a.sink, a.form,
-        (float*)a.partial);
+        (float*)a.partial, a.gate);
 }
 
 template <int KQ>
@@ -1208,11 +1230,12 @@ NI_EXPORT int ni_bias_attention_mfma(const void* qkv, int row_stride, const void
                                      int table_width, const void* tiles, int n_tiles, const void* positions, const void* bias,
                                      int distances, void* out, int H, int G, int dk, int dv, int page_size, float scale,
                                      float temp_coef, int temp_every, int heads_per_chunk, int window, int keep_first,
-                                     float out_scale, const void* sink, float softcap, int chunk, int maps, void* partial, int dtype,
-                                     hipStream_t stream) {
+                                     float out_scale, const void* sink, float softcap, int chunk, int maps, void* partial, const void* gate_rows,
+                                     int gate_stride, int gate_every, int dtype, hipStream_t stream) {
     // `partial` (float32 [T][H][dv + 2], or null): the rows are left there unfinished, as runs of one; no sink
     if (n_tiles <= 0) return 0;
-    if (window < 0 || keep_first < 0 || chunk < 0 || (chunk && window) || maps < 1 || G % maps || (partial && sink)) return -1;
+    if (window < 0 || keep_first < 0 || chunk < 0 || (chunk && window) || maps < 1 || G % maps || (partial && (sink || gate_rows))) return -1;
+    if (gate_rows && (gate_every < 1 || gate_stride < (H * dv + gate_every - 1) / gate_every || maps != 1)) return -1;
     const bool one_pool = kpool == vpool && dk == dv;
     if (!ni_bias_attention_mfma_rows(dk, dv, one_pool) || H % G || heads_per_chunk < 1 || heads_per_chunk > MROWS) return -1;
     const int group = H / G;
@@ -1223,7 +1246,7 @@ NI_EXPORT int ni_bias_attention_mfma(const void* qkv, int row_stride, const void
     dim3 grid(n_tiles, G, (group + heads_per_chunk - 1) / heads_per_chunk);
     const MfmaArgs args{qkv, row_stride, kpool, vpool, block_table, table_width, tiles, positions, bias, distances, out, H, G, dk, dv,
                         page_size, scale, temp_coef, temp_every, heads_per_chunk, k_pieces, v_pieces, window, keep_first, out_scale, sink,
-                        ScoreForm{softcap, chunk, maps}, partial};
+                        ScoreForm{softcap, chunk, maps}, partial, Gate{(const float*)gate_rows, gate_stride, gate_every}};
     hipError_t err;
     // bfloat16 rows in whole 16-byte pieces
     if (dtype == 1 && k_pieces && v_pieces && row_stride % 8 == 0 && reinterpret_cast<uintptr_t>(qkv) % 16 == 0) {

@@ -607,7 +607,7 @@ def bias_attention(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
                    temp_coef: float, temp_every: int, heads_per_chunk: int, n_runs: int = 1,
                    workspace: Optional[torch.Tensor] = None, waves: int = 4, window: Optional[int] = None, keep_first: int = 0,
                    out_scale: float = 1.0, sink: Optional[torch.Tensor] = None, softcap: Optional[float] = None,
-                   chunk: Optional[int] = None, maps: int = 1) -> torch.Tensor:
+                   chunk: Optional[int] = None, maps: int = 1, gate=None) -> torch.Tensor:
     """Causal attention of the query heads in the first ``H * dk`` columns of ``qkv`` over the paged cache.
     ``tiles`` int32 [n, 4]: (sequence, first row, tokens, -) with tokens * heads of a chunk <= 16, the tokens of a
     tile being consecutive ones of one sequence; ``positions`` int32 [T] the position of every row;
@@ -620,7 +620,8 @@ def bias_attention(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
     ``c tanh(s / c)``; ``chunk`` n: a query sees the keys of its own chunk of n positions alone (instead of a window).
     ``maps`` m > 1: ``kpool`` rows hold m keys side by side, ``H`` counts the query heads of all maps, which come in the
     order [kv head][map][head of the group].  ``out`` None: the rows are left in ``workspace`` unfinished, every run by
-    itself (:func:`merge_maps` takes them so), and the workspace is returned."""
+    itself (:func:`merge_maps` takes them so), and the workspace is returned.  ``gate`` (rows, col, every): output channel j
+    of a token is multiplied by ``sigmoid(rows[t, col + j // every])``, ``rows`` float32 [T, wide]."""
     T, width = qkv.shape
     pages, G, ps, dk, dv = _map_sizes(kpool, vpool, maps)
     _gpu(qkv, "qkv")
@@ -633,7 +634,7 @@ def bias_attention(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
     if out is not None:
         _gpu(out, "out", qkv.dtype, (T, H * dv))
     else:
-        _need(sink is None and out_scale == 1.0, "an unfinished row has no sink and no scale yet")
+        _need(sink is None and out_scale == 1.0 and gate is None, "an unfinished row has no sink, no scale and no gate yet")
     _need(chunk is None or (window is None and chunk >= 1), "chunks take a window's place")
     _gpu(positions, "positions", torch.int32, (T,))
     _need(H % G == 0 and H * dk <= width, "heads")
@@ -656,12 +657,24 @@ def bias_attention(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
                                                  _ptr(out), H, G, dk, dv, ps, _float(scale), _float(temp_coef), int(temp_every),
                                                  heads_per_chunk, n_runs, _ptr(workspace if n_runs > 1 or out is None else None), T, waves,
                                                  int(window or 0), int(keep_first), _float(out_scale), _ptr(sink),
-                                                 _float(softcap or 0.0), int(chunk or 0), maps, int(out is None),
+                                                 _float(softcap or 0.0), int(chunk or 0), maps, int(out is None), *_gate_args(gate, T, H * dv, maps),
                                                  dtype_code(qkv.dtype), _stream())
     if err == -2:
         raise KernelError(f"keys of {dk} and values of {dv} channels do not fit the kernel's staging memory")
     _check(err, "bias_attention")
     return workspace if out is None else out
+
+
+def _gate_args(gate, T: int, n: int, maps: int):
+    """(pointer, stride, every) of a gate ``(rows, col, every)`` on ``n`` output channels of T tokens, checked; None: none."""
+    if gate is None:
+        return _ptr(None), 0, 1
+    rows, col, every = gate
+    _gpu(rows, "gate rows", torch.float32)
+    _need(maps == 1, "the maps of a head are not gated one by one")
+    _need(every >= 1 and n % every == 0, "whole groups of channels share a gate")
+    _need(rows.dim() == 2 and rows.shape[0] == T and 0 <= col and col + n // every <= rows.shape[1], "the gate's columns lie outside its rows")
+    return ctypes.c_void_p(rows.data_ptr() + 4 * col), rows.shape[1], int(every)
 
 
 def _map_sizes(kpool: torch.Tensor, vpool: torch.Tensor, maps: int):
@@ -700,7 +713,7 @@ def bias_attention_mfma(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Ten
                         scale: float, temp_coef: float, temp_every: int, heads_per_chunk: int, window: Optional[int] = None,
                         keep_first: int = 0, out_scale: float = 1.0, sink: Optional[torch.Tensor] = None,
                         softcap: Optional[float] = None, chunk: Optional[int] = None, maps: int = 1,
-                        workspace: Optional[torch.Tensor] = None) -> torch.Tensor:
+                        workspace: Optional[torch.Tensor] = None, gate=None) -> torch.Tensor:
     """:func:`bias_attention` for steps with portions of prompts: tiles of up to 64 rows (tokens * heads of a chunk),
     both products on the float32 matrix instructions, the same formula and the same 32-bit softmax; no runs.  ``out``
     None: the rows are left in ``workspace`` (float32, T * H * (dv + 2)) unfinished, as runs of one."""
@@ -716,7 +729,7 @@ def bias_attention_mfma(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Ten
     if out is not None:
         _gpu(out, "out", qkv.dtype, (T, H * dv))
     else:
-        _need(sink is None and out_scale == 1.0, "an unfinished row has no sink and no scale yet")
+        _need(sink is None and out_scale == 1.0 and gate is None, "an unfinished row has no sink, no scale and no gate yet")
     _need(chunk is None or (window is None and chunk >= 1), "chunks take a window's place")
     _gpu(positions, "positions", torch.int32, (T,))
     _need(H % G == 0 and H * dk <= width, "heads")
@@ -739,6 +752,7 @@ def bias_attention_mfma(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Ten
                                                        _float(temp_coef), int(temp_every), heads_per_chunk,
                                                        int(window or 0), int(keep_first), _float(out_scale), _ptr(sink),
                                                        _float(softcap or 0.0), int(chunk or 0), maps,
-                                                       _ptr(workspace if out is None else None), dtype_code(qkv.dtype), _stream()),
+                                                       _ptr(workspace if out is None else None), *_gate_args(gate, T, H * dv, maps),
+                                                       dtype_code(qkv.dtype), _stream()),
            "bias_attention_mfma")
     return workspace if out is None else out

@@ -235,9 +235,6 @@ class LatentAttention(Part):
                                  adjacent=self.adjacent, q_dim=self.dq, rot_at_q=self.dk, queries_only=True)
         return q
 
-    def _gated(self, y, proj):
-        return K.gate_rows(y, proj, self.gate_col, every=self.dv if self.gate_per_head else 1)
-
     def forward(self, x, ctx, cache: LayerCache, out: Optional[torch.Tensor] = None):
         T, H = x.shape[0], self.H
         if cache.writes != self.own:
@@ -245,7 +242,7 @@ class LatentAttention(Part):
         proj = K.linear(x, self.w_in, out_dtype=torch.float32)
         q = self._queries(x, proj, ctx, cache)
         if self.always_expand or (self.expand_from is not None and not ctx.recording and ctx.max_q_len >= self.expand_from):
-            return K.linear(self._gated(self._over_heads(q, ctx, cache), proj), self.w_o, out_dtype=torch.float32, out=out)
+            return K.linear(self._over_heads(q, ctx, cache, proj), self.w_o, out_dtype=torch.float32, out=out)
         # the queries as the rows of the pages see them, [T, H * row]: a product per head, read and written in place
         seen = torch.empty(T, H * self.row, dtype=self.rt.dtype, device=x.device)
         torch.bmm(q.view(T, H, self.dq).transpose(0, 1), self.uk, out=seen.view(T, H, self.row).transpose(0, 1))
@@ -257,12 +254,12 @@ class LatentAttention(Part):
         y = K.gate_heads(heads, proj, self.gate_col, self.rt.dtype, per_head=self.gate_per_head)
         return K.linear(y, self.w_o, out_dtype=torch.float32, out=out)
 
-    def _over_heads(self, q, ctx, cache: LayerCache) -> torch.Tensor:
+    def _over_heads(self, q, ctx, cache: LayerCache, proj) -> torch.Tensor:
         """Attention with keys and values of every head written out: the pages that hold a key some token of the step
         can see are picked out of the pool, ``k = W_uk c`` (beside the rotated channels, the same for every head) and
         ``v = W_uv c`` are two products over them, laid out as pools of H heads, and the kernels walk them through a
         block table of their own that holds nothing else.  A tile of queries starts at the tile of 64 keys in which its
-        first token's window starts; the picked pages start there."""
+        first token's window starts; the picked pages start there.  The output is gated as its rows are finished."""
         ps, window = int(cache.kpool.shape[2]), self.window
         B, width = cache.block_table.shape
         pairs, table, at = [], np.full((B, width), -1, dtype=np.int32), 0
@@ -278,7 +275,7 @@ class LatentAttention(Part):
         latents = K.gather_pages(cache.kpool, cache.block_table, pairs_dev).view(at * ps, self.row)
         keys = K.rows_to_pages(K.linear(latents, self.uk_rows), ps, self.H, self.dq)
         values = K.rows_to_pages(K.linear(latents, self.uv_rows), ps, self.H, self.dv)
-        return self.heads(q, ctx, keys, values, table_dev, window)
+        return self.heads(q, ctx, keys, values, table_dev, window, gate=(proj, self.gate_col, self.dv if self.gate_per_head else 1))
 
 
 # ------------------------------------------------------------------ matrix memory with exponential gates

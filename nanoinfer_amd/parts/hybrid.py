@@ -200,15 +200,18 @@ class PagedSoftmax:
         self.wide_heads = min(group, wide) if wide else 0
         self.wide_tokens = max(1, wide // self.wide_heads) if wide else 0
 
-    def __call__(self, qkv, ctx, kpool, vpool, block_table, window: Optional[int] = None, keep_first: int = 0, out_scale: float = 1.0):
-        return self._run(qkv, ctx, kpool, vpool, block_table, window, keep_first, out_scale, True)[0]
+    def __call__(self, qkv, ctx, kpool, vpool, block_table, window: Optional[int] = None, keep_first: int = 0, out_scale: float = 1.0,
+                 gate=None):
+        """``gate`` (rows, col, every): output channel j of a token is multiplied by ``sigmoid(rows[t, col + j // every])`` as
+        its row is finished."""
+        return self._run(qkv, ctx, kpool, vpool, block_table, window, keep_first, out_scale, True, gate)[0]
 
     def unfinished(self, qkv, ctx, kpool, vpool, block_table, window: Optional[int] = None, keep_first: int = 0):
         """``(rows, runs)``: the attention's rows as the kernels leave them before they are finished (float32 [T, H, runs,
         dv + 2]: maximum, sum, weighted sum of every run of keys), for a kernel that finishes them in its own way."""
         return self._run(qkv, ctx, kpool, vpool, block_table, window, keep_first, 1.0, False)
 
-    def _run(self, qkv, ctx, kpool, vpool, block_table, window, keep_first, out_scale, finish: bool):
+    def _run(self, qkv, ctx, kpool, vpool, block_table, window, keep_first, out_scale, finish: bool, gate=None):
         T = qkv.shape[0]
         out = torch.empty(T, self.H * self.dv, dtype=qkv.dtype, device=qkv.device) if finish else None
         if self.wide_heads and ctx.max_q_len >= K.BIAS_ATTENTION_MFMA_FROM:
@@ -218,7 +221,7 @@ class PagedSoftmax:
             ws = None if finish else ctx.workspace(T * self.H * (self.dv + 2))
             return K.bias_attention_mfma(qkv, kpool, vpool, block_table, tiles, ctx.positions, self.bias, out, self.H,
                                          self.scale, self.temp_coef, self.temp_every, self.wide_heads, window, keep_first, out_scale,
-                                         sink=self.sink, workspace=ws, **self.extras), 1
+                                         sink=self.sink, workspace=ws, gate=gate, **self.extras), 1
         tiles = ctx.q_tiles(self.tile_tokens)
         if tiles is None:
             raise K.KernelError("this step was recorded without the tiles of its tokens")
@@ -236,7 +239,7 @@ class PagedSoftmax:
         ws = ctx.workspace(T * self.H * runs * (self.dv + 2)) if runs > 1 or not finish else None
         return K.bias_attention(qkv, kpool, vpool, block_table, tiles, ctx.positions, self.bias, out, self.H,
                                 self.scale, self.temp_coef, self.temp_every, self.heads_per_chunk, runs, ws, waves, window,
-                                keep_first, out_scale, sink=self.sink, **self.extras), runs
+                                keep_first, out_scale, sink=self.sink, gate=gate, **self.extras), runs
 
 
 @register_part("mixer", "bias_attention")
@@ -299,11 +302,11 @@ class BiasAttention(Part):
             K.kv_store(qkv, self.H * self.dk, (self.H + self.G) * self.dk, cache.slot_mapping, cache.kpool, cache.vpool)
         return K.linear(self.attend(qkv, ctx, cache), self.w_o, out_dtype=torch.float32)
 
-    def attend(self, qkv, ctx, cache: LayerCache, window: Optional[int] = None, keep_first: int = 0, out_scale: float = 1.0):
+    def attend(self, qkv, ctx, cache: LayerCache, window: Optional[int] = None, keep_first: int = 0, out_scale: float = 1.0, gate=None):
         """The queries in the first ``H * dk`` columns of ``qkv`` over the keys and values of the cache: [T, H * dv] in
         the compute type.  ``window`` n: a query sees its last n keys and the sequence's first ``keep_first``;
-        ``out_scale`` multiplies the result."""
-        return self.core(qkv, ctx, cache.kpool, cache.vpool, cache.block_table, window, keep_first, out_scale)
+        ``out_scale`` multiplies the result; ``gate``: see :class:`PagedSoftmax`."""
+        return self.core(qkv, ctx, cache.kpool, cache.vpool, cache.block_table, window, keep_first, out_scale, gate)
 
 
 # ------------------------------------------------------------------ gated delta rule, a decay per key channel

@@ -104,8 +104,7 @@ class SinkAttention(WindowAttention):
         else:
             K.qk_norm_rope_store(proj, ctx.positions, cache.slot_mapping, self.head_q_norm, self.head_k_norm, self.eps, self.freq,
                                  self.amplitude, q, cache.kpool, cache.vpool, self.H, per_head=True, adjacent=self.adjacent)
-        attended = self.attend(q, ctx, cache, self.window, 0, 1.0)
-        gated = K.gate_rows(attended, proj, self.gate_col, out=attended, every=self.gate_every)
+        gated = self.attend(q, ctx, cache, self.window, 0, 1.0, gate=(proj, self.gate_col, self.gate_every))
         return K.linear(gated, self.w_o, out_dtype=torch.float32, out=out)
 
 

@@ -279,7 +279,7 @@ def test_far_keys_the_sink_and_the_query_factor_in_both_attention_kernels(H, G, 
     heads' sinks (which run from no weight to most of it), so a sink that is left out, counted a run too often or scaled
     shows in every row, and so does a query factor that steps one position off.  Prompt portions (the matrix cores where
     they take the sizes, else the vector units) and single tokens with the keys cut into runs must both give the
-    written-out softmax."""
+    written-out softmax, as it is, with a gate a channel and with a gate a head."""
     from nanoinfer_amd import kernels as K
     from nanoinfer_amd.kernels import stream
     dev = torch.device("cuda")
@@ -305,6 +305,10 @@ def test_far_keys_the_sink_and_the_query_factor_in_both_attention_kernels(H, G, 
         return torch.from_numpy(out.reshape(T, -1))
 
     want = written_out(factor)
+    before = 3                                        # columns that belong to nobody
+    gates = torch.randn(T, before + H * dv + 2, generator=g)
+    factors = {None: 1.0, 1: torch.sigmoid(gates[:, before:before + H * dv].double()),
+               dv: torch.sigmoid(gates[:, before:before + H].double()).repeat_interleave(dv, dim=1)}
     if temp is not None and temp[1] > 1:                                  # rows do depend on where the factor steps
         shifted = P.temperature(np.arange(T) - 1, dict(zip(("coef", "every"), temp)))
         moved = (written_out(shifted) - want).abs().max(dim=1).values / want.abs().max()
@@ -325,9 +329,13 @@ def test_far_keys_the_sink_and_the_query_factor_in_both_attention_kernels(H, G, 
     tol = 2e-5 if dtype == torch.float32 else 2e-2
     group = H // G
 
-    def check(out, rows, what):
-        err = float((out.double().cpu() - want[rows]).abs().max() / want.abs().max())
-        assert err <= tol, f"{what}: {err:.3e}"
+    def gate(rows, every):
+        return None if every is None else (gates[rows].contiguous().to(dev), before, every)
+
+    def check(out, rows, every, what):
+        full = want * factors[every]
+        err = float((out.double().cpu() - full[rows]).abs().max() / full.abs().max())
+        assert err <= tol, f"{what}, gate every {every}: {err:.3e}"
 
     for start in (0, 100, 203):
         n = T - start
@@ -337,23 +345,24 @@ def test_far_keys_the_sink_and_the_query_factor_in_both_attention_kernels(H, G, 
                 continue
             heads = min(group, rows_per)
             tiles = torch.tensor(K.build_q_tiles([0], [n], [T], max(1, rows_per // heads)), dtype=torch.int32).view(-1, 4).to(dev)
-            out = torch.empty(n, H * dv, dtype=dtype, device=dev)
             fn = stream.bias_attention_mfma if wide else stream.bias_attention
-            fn(qrows[start:].contiguous(), kpool, vpool, pages, tiles, positions[start:].contiguous(), None, out, H, scale, coef, every,
-               heads, sink=sink_dev)
-            check(out, slice(start, T), f"portion from {start}, {'matrix cores' if wide else 'vector units'}")
+            for per in (None, 1, dv):
+                out = torch.empty(n, H * dv, dtype=dtype, device=dev)
+                fn(qrows[start:].contiguous(), kpool, vpool, pages, tiles, positions[start:].contiguous(), None, out, H, scale, coef, every,
+                   heads, sink=sink_dev, gate=gate(slice(start, T), per))
+                check(out, slice(start, T), per, f"portion from {start}, {'matrix cores' if wide else 'vector units'}")
     heads = min(group, stream.bias_attention_rows())
     edges = [] if not every else [m * every + o for m in (1, 2) for o in (-2, -1, 0)]
     for pos in [0, 1, 63, 64, 65, 127, 128, 200, 299] + edges:
         if not 0 <= pos < T:
             continue
         tiles = torch.tensor(K.build_q_tiles([0], [1], [pos + 1], 1), dtype=torch.int32).view(-1, 4).to(dev)
-        for runs in (1, 3, 8):
+        for runs, per in ((1, None), (1, 1), (3, None), (3, dv), (8, 1), (8, dv)):
             out = torch.empty(1, H * dv, dtype=dtype, device=dev)
             ws = torch.empty(H * runs * (dv + 2), dtype=torch.float32, device=dev) if runs > 1 else None
             stream.bias_attention(qrows[pos:pos + 1].contiguous(), kpool, vpool, pages, tiles, positions[pos:pos + 1].contiguous(), None,
-                                  out, H, scale, coef, every, heads, runs, ws, 4, sink=sink_dev)
-            check(out, slice(pos, pos + 1), f"single token at {pos} in {runs} runs")
+                                  out, H, scale, coef, every, heads, runs, ws, 4, sink=sink_dev, gate=gate(slice(pos, pos + 1), per))
+            check(out, slice(pos, pos + 1), per, f"single token at {pos} in {runs} runs")
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
