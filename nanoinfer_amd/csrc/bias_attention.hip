@@ -221,6 +221,131 @@ qk_norm_rope_store_kernel(const float* __restrict__ proj, int row_stride, const 
     }
 }
 
+// The same with norms a head (or none), for heads of up to 64 SL channels: a wavefront takes HB heads at once, whose channels
+// lie in its lanes (channel lane + 64 u in slot u), so a head is read once, normed, rotated through the wavefront's own LDS
+// and stored; what the HB heads wait for they wait for together.
+template <typename T, int SL, int HB>
+__global__ void __launch_bounds__(256)
+qk_heads_kernel(const float* __restrict__ proj, int row_stride, const int32_t* __restrict__ positions,
+                const int32_t* __restrict__ slot_mapping, const float* __restrict__ wq, const float* __restrict__ wk,
+                float eps, const float* __restrict__ freq, float amplitude, T* __restrict__ q_out,
+                T* __restrict__ kpool, T* __restrict__ vpool, int page_size, QkForm f) {
+    __shared__ float cos_of[ROT_PAIRS], sin_of[ROT_PAIRS];
+    __shared__ float turned[4][HB][64 * SL];
+    const int t = blockIdx.x, tid = threadIdx.x, lane = tid & (WAVE - 1), wave = tid / WAVE;
+    const float* row = proj + static_cast<size_t>(t) * row_stride;
+    const int H = f.H, G = f.G, dq = f.dq, dk = f.dk, dv = f.dv, half = f.rot / 2;
+    const int slices = gridDim.y, slice = blockIdx.y;
+    if (freq) {
+        const float pos = static_cast<float>(positions[t]);
+        for (int p = tid; p < half; p += blockDim.x) {
+            float sn, cs;
+            sincosf(pos * freq[p], &sn, &cs);
+            cos_of[p] = cs * amplitude;
+            sin_of[p] = sn * amplitude;
+        }
+        __syncthreads();
+    }
+    const int slot = slot_mapping ? slot_mapping[t] : -1;
+    const int page = slot >= 0 ? slot / page_size : 0, in_page = slot >= 0 ? slot % page_size : 0;
+    float weight_q[SL], weight_k[SL];
+#pragma unroll
+    for (int u = 0; u < SL; ++u) {
+        const int c = lane + 64 * u;
+        weight_q[u] = wq && c < dq ? wq[c] : 0.f;
+        weight_k[u] = wk && c < f.k_normed ? wk[c] : 0.f;
+    }
+    const int per = (H + G + slices - 1) / slices, first = slice * per, last = min(H + G, first + per);
+    for (int base = first + wave * HB; base < last; base += 4 * HB) {
+        float x[HB][SL], ss[HB];
+#pragma unroll
+        for (int b = 0; b < HB; ++b) {
+            const int hd = min(base + b, last - 1);              // (a head too many is read again and not stored)
+            const bool is_q = hd < H;
+            const float* src = is_q ? row + hd * dq : row + H * dq + (hd - H) * dk;
+            const int n = is_q ? dq : dk;
+#pragma unroll
+            for (int u = 0; u < SL; ++u) x[b][u] = lane + 64 * u < n ? src[lane + 64 * u] : 0.f;
+        }
+#pragma unroll
+        for (int b = 0; b < HB; ++b) {
+            const int normed = min(base + b, last - 1) < H ? dq : f.k_normed;
+            ss[b] = 0.f;
+#pragma unroll
+            for (int u = 0; u < SL; ++u) ss[b] += lane + 64 * u < normed ? x[b][u] * x[b][u] : 0.f;
+        }
+#pragma unroll
+        for (int b = 0; b < HB; ++b) ss[b] = wave_sum(ss[b]);
+#pragma unroll
+        for (int b = 0; b < HB; ++b) {
+            const bool is_q = min(base + b, last - 1) < H;
+            const int normed = !(is_q ? wq : wk) ? 0 : is_q ? dq : f.k_normed;
+            const float r = normed > 0 ? 1.0f / sqrtf(ss[b] / static_cast<float>(normed) + eps) : 1.f;
+#pragma unroll
+            for (int u = 0; u < SL; ++u)
+                if (lane + 64 * u < normed) x[b][u] = x[b][u] * r * (is_q ? weight_q[u] : weight_k[u]);
+        }
+        if (freq) {
+            __builtin_amdgcn_wave_barrier();      // a wavefront reads only what it wrote itself, and its LDS accesses stay in order
+#pragma unroll
+            for (int b = 0; b < HB; ++b)
+#pragma unroll
+                for (int u = 0; u < SL; ++u) turned[wave][b][lane + 64 * u] = x[b][u];
+            __builtin_amdgcn_wave_barrier();
+#pragma unroll
+            for (int b = 0; b < HB; ++b) {
+                const int at = min(base + b, last - 1) < H ? f.rot_at_q : f.rot_at_k;
+#pragma unroll
+                for (int u = 0; u < SL; ++u) {
+                    const int cr = lane + 64 * u - at;
+                    if (cr >= 0 && cr < f.rot) {
+                        const bool one = f.adjacent ? !(cr & 1) : cr < half;
+                        const int partner = f.adjacent ? (cr ^ 1) : (one ? cr + half : cr - half);
+                        const int p = f.adjacent ? (cr >> 1) : (one ? cr : cr - half);
+                        const float other = turned[wave][b][at + partner], cs = cos_of[p], sn = sin_of[p];
+                        x[b][u] = one ? x[b][u] * cs - other * sn : x[b][u] * cs + other * sn;
+                    }
+                }
+            }
+        }
+#pragma unroll
+        for (int b = 0; b < HB; ++b) {
+            const int hd = base + b;
+            if (hd >= last || (hd >= H && slot < 0)) continue;
+            T* dst = hd < H ? q_out + (static_cast<size_t>(t) * H + hd) * dq
+                            : kpool + ((static_cast<size_t>(page) * G + (hd - H)) * page_size + in_page) * dk;
+            const int n = hd < H ? dq : dk;
+#pragma unroll
+            for (int u = 0; u < SL; ++u)
+                if (lane + 64 * u < n) st(dst + lane + 64 * u, x[b][u]);
+        }
+    }
+    if (slot >= 0) {
+        const float* vsrc = row + H * dq + (f.v_from_k ? 0 : G * dk);      // the values may be the keys as projected
+        const int vper = (G * dv + slices - 1) / slices;
+        for (int i = slice * vper + tid; i < min(G * dv, (slice + 1) * vper); i += blockDim.x) {
+            const int g = i / dv, c = i - g * dv;
+            st(vpool + ((static_cast<size_t>(page) * G + g) * page_size + in_page) * dv + c, vsrc[i]);
+        }
+    }
+}
+
+template <typename T>
+static void launch_qk_heads(const float* proj, int row_stride, const int32_t* positions, const int32_t* slot_mapping, const float* wq,
+                            const float* wk, float eps, const float* freq, float amplitude, T* q_out, T* kpool, T* vpool, int page_size,
+                            const QkForm& f, int Tn, hipStream_t stream) {
+    const int size = std::max(f.H > 0 ? f.dq : 0, f.G > 0 ? f.dk : 0);
+    // few tokens: one head a wavefront; many: every workgroup a row of its own, as long as that fills the chip
+    const int slices = std::max(1, std::min({16, (f.H + f.G + 3) / 4, 2048 / std::max(Tn, 1)}));
+    const dim3 grid(Tn, slices);
+    if (size <= 64)
+        qk_heads_kernel<T, 1, 4><<<grid, 256, 0, stream>>>(proj, row_stride, positions, slot_mapping, wq, wk, eps, freq, amplitude, q_out, kpool, vpool, page_size, f);
+    else if (size <= 128)
+        qk_heads_kernel<T, 2, 2><<<grid, 256, 0, stream>>>(proj, row_stride, positions, slot_mapping, wq, wk, eps, freq, amplitude, q_out, kpool, vpool, page_size, f);
+    else
+        qk_heads_kernel<T, 4, 2><<<grid, 256, 0, stream>>>(proj, row_stride, positions, slot_mapping, wq, wk, eps, freq, amplitude, q_out, kpool, vpool, page_size, f);
+}
+
 // `per_head`, `adjacent`, `dq`, `k_normed`, `rot_at_q`, `rot_at_k`: see the kernel.  G may be 0 (queries alone).
 NI_EXPORT int ni_qk_norm_rope_store(const void* proj, int row_stride, const void* positions, const void* slot_mapping,
                                     const void* wq, const void* wk, float eps, const void* freq, int rot, float amplitude,
@@ -237,6 +362,16 @@ NI_EXPORT int ni_qk_norm_rope_store(const void* proj, int row_stride, const void
     if (per_head && H + G > NORM_HEADS) return -1;
     if ((H > 0 && !q_out) || (G > 0 && slot_mapping && (!kpool || (dv > 0 && !vpool)))) return -1;
     const QkForm f{H, G, dq, dk, dv, k_normed, freq ? rot : 0, rot_at_q, rot_at_k, v_from_k != 0, per_head != 0, adjacent != 0};
+    if ((per_head || (!wq && !wk)) && std::max(H > 0 ? dq : 0, G > 0 ? dk : 0) <= 4 * WAVE) {
+        if (dtype == 0)
+            launch_qk_heads<float>((const float*)proj, row_stride, (const int32_t*)positions, (const int32_t*)slot_mapping, (const float*)wq,
+                                   (const float*)wk, eps, (const float*)freq, amplitude, (float*)q_out, (float*)kpool, (float*)vpool, page_size, f, T, stream);
+        else
+            launch_qk_heads<bf16_t>((const float*)proj, row_stride, (const int32_t*)positions, (const int32_t*)slot_mapping, (const float*)wq,
+                                    (const float*)wk, eps, (const float*)freq, amplitude, (bf16_t*)q_out, (bf16_t*)kpool, (bf16_t*)vpool, page_size, f, T,
+                                    stream);
+        return NI_LAUNCH_RESULT();
+    }
     // few tokens: a row's elements over several workgroups, one pass of 256 threads each
     const int slices = T >= 64 ? 1 : std::max(1, std::min(16, (H * dq + G * dk + 255) / 256));
     const dim3 grid(T, slices);
@@ -969,6 +1104,205 @@ bias_attention_bf16_kernel(const bf16_t* __restrict__ qkv, int row_stride, const
     }
 }
 
+// ------------------------------------------------------------------ single tokens and short portions in bfloat16
+// The tiles of the vector-unit kernel (up to 16 rows of (token, head), one run of keys a workgroup) with the products of
+// the kernel above.  Sixteen rows are one operand of an MFMA, so the four wavefronts share the run's keys instead of its
+// rows: wavefront w takes the units of 32 keys w, w + 4, .., each with a maximum, sum and weighted sum of its own, which
+// meet in LDS at the end.  Keys come from their pages straight into the first operand's registers (a lane: 8 channels of
+// one key, 16 bytes); values go through a tile of the wavefront's own in LDS for the transposing reads, which needs no
+// barrier.  The next unit's keys and values are asked for before the softmax of this one.
+#define UNIT 32
+
+template <int KQ, int DVB>
+__global__ void __launch_bounds__(WAVES * WAVE)
+bias_attention_bf16_token_kernel(const bf16_t* __restrict__ qkv, int row_stride, const bf16_t* __restrict__ kpool, const bf16_t* __restrict__ vpool,
+                                 const int32_t* __restrict__ block_table, int table_width, const int32_t* __restrict__ tiles,
+                                 const int32_t* __restrict__ positions, const float* __restrict__ bias, int distances, bf16_t* __restrict__ out,
+                                 int H, int G, int dk, int dv, int page_size, float scale, float temp_coef, int temp_every, int heads_per_chunk,
+                                 int n_runs, float* __restrict__ partial, int window, int keep_first, float out_scale,
+                                 const float* __restrict__ sink, ScoreForm form, Gate gate) {
+    constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
+    constexpr int VROW = 16 * DVB + TILE_PAD, MROW = 16 * DVB;
+    constexpr int TILE_BYTES = WAVES * UNIT * VROW * 2, MEET_BYTES = WAVES * ROWS * MROW * 4;
+    __shared__ __attribute__((aligned(16))) unsigned char staged[TILE_BYTES > MEET_BYTES ? TILE_BYTES : MEET_BYTES];
+    __shared__ float meet_m[WAVES][ROWS], meet_l[WAVES][ROWS];
+    const int tile = blockIdx.x / n_runs, run = blockIdx.x % n_runs, g = blockIdx.y, chunk = blockIdx.z;
+    const int seq = tiles[4 * tile], first_row = tiles[4 * tile + 1], n_tok = tiles[4 * tile + 2];
+    const int first_pos = positions[first_row];
+    const int group = H / G;
+    const int heads_here = std::min(heads_per_chunk, group - chunk * heads_per_chunk);
+    const int head0 = g * group + chunk * heads_per_chunk;
+    const int n_rows = n_tok * heads_here;        // row r = token r / heads_here, head r % heads_here
+    const int tid = threadIdx.x, lane = tid & (WAVE - 1), wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+    const int i = lane & 15, kg = lane >> 4;
+    const int kv = g / form.maps, kv_heads = G / form.maps, k_row = form.maps * dk;
+    kpool += (g % form.maps) * dk;
+    uint16_t* Vs = reinterpret_cast<uint16_t*>(staged) + wave * UNIT * VROW;
+
+    const bool valid = i < n_rows;
+    const int token = valid ? i / heads_here : 0;
+    const int pos = first_pos + token;
+    const int head = head0 + (valid ? i % heads_here : 0);
+    const int lo = first_seen(pos, window, form.chunk);
+    const int steps = temp_every > 0 ? (pos + 1) / temp_every : 0;
+    const float factor = scale * (1.0f + temp_coef * logf(static_cast<float>(steps) + 1.0f));
+    const float cap2 = form.softcap * LOG2E, cap_in = form.softcap > 0.f ? 2.0f * LOG2E / form.softcap : 0.f;      // as in the kernel above
+    uint4 qf[KQ];
+#pragma unroll
+    for (int kk = 0; kk < KQ; ++kk) {
+        const int c = 32 * kk + 8 * kg;
+        qf[kk] = valid && c < dk ? *reinterpret_cast<const uint4*>(qkv + static_cast<size_t>(first_row + token) * row_stride + head * dk + c)
+                                 : make_uint4(0u, 0u, 0u, 0u);
+    }
+    float m = -INFINITY, l = 0.f;                 // of row i; the maximum in units of log2
+    floatx4_t acc[DVB];
+#pragma unroll
+    for (int db = 0; db < DVB; ++db) acc[db] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+    const int dvb = dv / 16, v_pieces = dv / 8;
+    const int last_pos = first_pos + n_tok - 1;
+    const int last_lo = first_seen(last_pos, window, form.chunk);      // the latest first key of any row
+    const int32_t* table = block_table + static_cast<size_t>(seq) * table_width;
+    const KeyWalk walk(first_pos, last_pos, window, keep_first, form.chunk);
+    const int per_run = (walk.steps + n_runs - 1) / n_runs;            // tiles of KEYS keys a run
+    const int v0 = run * per_run, n_units = std::max(0, std::min(walk.steps, v0 + per_run) - v0) * (KEYS / UNIT);
+    auto unit_key = [&](int u) { return walk.first_key(v0 + u / (KEYS / UNIT)) + u % (KEYS / UNIT) * UNIT; };
+    uint4 kr[UNIT / 16][KQ], vr[DVB];
+    auto page_of = [&](int key) { return key <= last_pos ? table[key / page_size] : -1; };
+    auto ask = [&](int k0) {
+#pragma unroll
+        for (int j = 0; j < UNIT / 16; ++j) {
+            const int key = k0 + 16 * j + i, page = page_of(key);
+            const bf16_t* src = kpool + ((static_cast<size_t>(std::max(page, 0)) * kv_heads + kv) * page_size + key % page_size) * k_row + 8 * kg;
+#pragma unroll
+            for (int kk = 0; kk < KQ; ++kk)
+                kr[j][kk] = page >= 0 && 32 * kk + 8 * kg < dk ? *reinterpret_cast<const uint4*>(src + 32 * kk) : make_uint4(0u, 0u, 0u, 0u);
+        }
+#pragma unroll
+        for (int u = 0; u < DVB; ++u) {           // UNIT rows of v_pieces 16-byte pieces, a piece a lane: dv / 16 times
+            vr[u] = make_uint4(0u, 0u, 0u, 0u);
+            if (u < dvb) {
+                const int idx = u * WAVE + lane, j = idx / v_pieces, key = k0 + j, page = page_of(key);
+                if (page >= 0)
+                    vr[u] = *reinterpret_cast<const uint4*>(vpool + ((static_cast<size_t>(page) * kv_heads + kv) * page_size + key % page_size) * dv +
+                                                            (idx - j * v_pieces) * 8);
+            }
+        }
+    };
+    if (wave < n_units) ask(unit_key(wave));
+    for (int u = wave; u < n_units; u += WAVES) {
+        const int k0 = unit_key(u);
+        floatx4_t sc[UNIT / 16];
+#pragma unroll
+        for (int j = 0; j < UNIT / 16; ++j) {
+            sc[j] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KQ; ++kk)
+                if (32 * kk < dk)
+                    sc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kr[j][kk]), __builtin_bit_cast(bf16x8_t, qf[kk]),
+                                                                    sc[j], 0, 0, 0);
+        }
+        __builtin_amdgcn_wave_barrier();          // the reads of the unit before come first (one wavefront's LDS accesses stay in order)
+#pragma unroll
+        for (int x = 0; x < DVB; ++x) {
+            if (x < dvb) {
+                const int idx = x * WAVE + lane, j = idx / v_pieces;
+                *reinterpret_cast<uint4*>(Vs + j * VROW + (idx - j * v_pieces) * 8) = vr[x];
+            }
+        }
+        __builtin_amdgcn_wave_barrier();
+        if (u + WAVES < n_units) ask(unit_key(u + WAVES));
+        float top = -INFINITY;
+#pragma unroll
+        for (int j = 0; j < UNIT / 16; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                float s = sc[j][r] * factor;
+                if (bias) {
+                    const int back = std::min(std::max(pos - (k0 + 16 * j + 4 * kg + r), 0), distances - 1);
+                    s += bias[static_cast<size_t>(back) * H + head];
+                }
+                sc[j][r] = form.softcap > 0.f ? cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * cap_in) + 1.0f) : s * LOG2E;
+            }
+        if (k0 + UNIT - 1 > first_pos || k0 < last_lo) {       // some row does not see every key of the unit
+#pragma unroll
+            for (int j = 0; j < UNIT / 16; ++j)
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (!key_seen(k0 + 16 * j + 4 * kg + r, pos, lo, keep_first)) sc[j][r] = -INFINITY;
+        }
+#pragma unroll
+        for (int j = 0; j < UNIT / 16; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) top = fmaxf(top, sc[j][r]);
+        top = groups4(top, true);
+        const float m_new = fmaxf(m, top);
+        const float m_ref = m_new > -INFINITY ? m_new : 0.f;   // a row that has seen no key yet: weights 2^-inf = 0
+        const float alpha = __builtin_amdgcn_exp2f(m - m_ref); // 0 at the row's first keys
+        float sum = 0.f;
+        uint32_t hi[UNIT / 16][2], rest[UNIT / 16][2];         // the weights as pairs: upper halves, what they leave
+#pragma unroll
+        for (int j = 0; j < UNIT / 16; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; r += 2) {
+                const float p0 = __builtin_amdgcn_exp2f(sc[j][r] - m_ref), p1 = __builtin_amdgcn_exp2f(sc[j][r + 1] - m_ref);
+                sum += p0 + p1;
+                const uint32_t u0 = __float_as_uint(p0), u1 = __float_as_uint(p1);
+                hi[j][r / 2] = (u0 >> 16) | (u1 & 0xffff0000u);
+                rest[j][r / 2] = pack_bf16x2(p0 - __uint_as_float(u0 & 0xffff0000u), p1 - __uint_as_float(u1 & 0xffff0000u));
+            }
+        l = l * alpha + groups4(sum, false);
+        m = m_new;
+        const bf16x8_t p_hi = __builtin_bit_cast(bf16x8_t, make_uint4(hi[0][0], hi[0][1], hi[1][0], hi[1][1]));
+        const bf16x8_t p_rest = __builtin_bit_cast(bf16x8_t, make_uint4(rest[0][0], rest[0][1], rest[1][0], rest[1][1]));
+#pragma unroll
+        for (int db = 0; db < DVB; ++db) {
+            if (db < dvb) {
+                const bf16x8_t vt = read_values_t(Vs, VROW, 16 * db, i, kg);
+                floatx4_t a = acc[db] * alpha;
+                a = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, p_hi, a, 0, 0, 0);
+                acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, p_rest, a, 0, 0, 0);
+            }
+        }
+    }
+    // the wavefronts' rows meet: a lane has dims 16 db + 4 kg .. of row i
+    __syncthreads();
+    float* meet = reinterpret_cast<float*>(staged);
+#pragma unroll
+    for (int db = 0; db < DVB; ++db)
+        if (db < dvb)
+            *reinterpret_cast<float4*>(meet + (wave * ROWS + i) * MROW + 16 * db + 4 * kg) = make_float4(acc[db][0], acc[db][1], acc[db][2], acc[db][3]);
+    if (kg == 0) {
+        meet_m[wave][i] = m;
+        meet_l[wave][i] = l;
+    }
+    __syncthreads();
+    for (int e = tid; e < n_rows * dv; e += WAVES * WAVE) {
+        const int r = e / dv, c = e - r * dv, t = first_row + r / heads_here, hd = head0 + r % heads_here;
+        float M = meet_m[0][r], L = 0.f, a = 0.f;
+#pragma unroll
+        for (int w = 1; w < WAVES; ++w) M = fmaxf(M, meet_m[w][r]);
+        const float ref = M > -INFINITY ? M : 0.f;
+#pragma unroll
+        for (int w = 0; w < WAVES; ++w) {
+            const float f = __builtin_amdgcn_exp2f(meet_m[w][r] - ref);
+            L += f * meet_l[w][r];
+            a += f * meet[(w * ROWS + r) * MROW + c];
+        }
+        if (partial) {
+            float* prow = partial + ((static_cast<size_t>(t) * H + hd) * n_runs + run) * (dv + 2);
+            if (c == 0) { prow[0] = M * LN2; prow[1] = L; }
+            prow[2 + c] = a;
+            continue;
+        }
+        float inv = out_scale / L;
+        if (sink) {             // one more term in the denominator, as in the kernels above
+            const float sk = sink[hd] * LOG2E, top = fmaxf(M, sk), f = __builtin_amdgcn_exp2f(M - top);
+            inv = out_scale * f / (L * f + __builtin_amdgcn_exp2f(sk - top));
+        }
+        st(out + static_cast<size_t>(t) * (H * dv) + hd * dv + c, a * inv * gate.of(t, hd * dv + c));
+    }
+}
+
 // out[row, :] = sum_r acc_r e^(m_r - M) / (sum_r l_r e^(m_r - M) + e^(sink - M)) over the runs of a row (an empty run
 // has l = 0; no sink: no such term; M is the maximum over the runs and the sink).
 // The weights e^(m_r - M) go through LDS, and the sums over the runs then read nothing that depends on an earlier read.
@@ -1118,6 +1452,34 @@ NI_EXPORT int ni_kv_store(const void* qkv, int row_stride, int k_off, int v_off,
     return NI_LAUNCH_RESULT();
 }
 
+struct MfmaArgs {
+    const void *qkv; int row_stride; const void *kpool, *vpool, *block_table; int table_width; const void *tiles, *positions, *bias;
+    int distances; void* out; int H, G, dk, dv, page_size; float scale, temp_coef; int temp_every, heads_per_chunk;
+    bool k_pieces, v_pieces; int window, keep_first; float out_scale; const void* sink; ScoreForm form; void* partial; Gate gate;
+};
+
+// Sizes that the kernel for single tokens and short portions in bfloat16 takes: rows of whole 16-byte pieces, values in blocks
+// of 16 channels
+static bool bf16_tokens(int dk, int dv) { return dk % 8 == 0 && dk >= 8 && dk <= 256 && dv % 16 == 0 && dv >= 16 && dv <= 256; }
+
+NI_EXPORT int ni_bias_attention_bf16_tokens(int dk, int dv) { return bf16_tokens(dk, dv); }
+
+template <int KQ, int DVB>
+static void launch_tokens(const MfmaArgs& a, int n_runs, dim3 grid, hipStream_t stream) {
+    bias_attention_bf16_token_kernel<KQ, DVB><<<grid, WAVES * WAVE, 0, stream>>>(
+        (const bf16_t*)a.qkv, a.row_stride, (const bf16_t*)a.kpool, (const bf16_t*)a.vpool, (const int32_t*)a.block_table, a.table_width,
+        (const int32_t*)a.tiles, (const int32_t*)a.positions, (const float*)a.bias, a.distances, (bf16_t*)a.out, a.H, a.G, a.dk, a.dv,
+        a.page_size, a.scale, a.temp_coef, a.temp_every, a.heads_per_chunk, n_runs, (float*)a.partial, a.window, a.keep_first, a.out_scale,
+        (const float*)a.sink, a.form, a.gate);
+}
+
+template <int KQ>
+static void launch_tokens_values(const MfmaArgs& a, int n_runs, dim3 grid, hipStream_t stream) {
+    if (a.dv <= 64) launch_tokens<KQ, 4>(a, n_runs, grid, stream);
+    else if (a.dv <= 128) launch_tokens<KQ, 8>(a, n_runs, grid, stream);
+    else launch_tokens<KQ, 16>(a, n_runs, grid, stream);
+}
+
 NI_EXPORT int ni_bias_attention_rows() { return ROWS; }
 
 NI_EXPORT int ni_bias_attention(const void* qkv, int row_stride, const void* kpool, const void* vpool, const void* block_table,
@@ -1158,6 +1520,16 @@ NI_EXPORT int ni_bias_attention(const void* qkv, int row_stride, const void* kpo
             (const float*)sink, form, gate);
         if (partial && !unfinished) merge_runs_kernel<float><<<n_rows * H, std::min(MAX_VCHUNKS, (dv + WAVE - 1) / WAVE) * WAVE, 0, stream>>>((const float*)partial, (float*)out, n_runs, dv, out_scale,
                                                                              (const float*)sink, H, gate);
+    } else if (bf16_tokens(dk, dv) && k_pieces && v_pieces && row_stride % 8 == 0 && reinterpret_cast<uintptr_t>(qkv) % 16 == 0) {
+        const MfmaArgs args{qkv, row_stride, kpool, vpool, block_table, table_width, tiles, positions, bias, distances, out, H, G, dk, dv,
+                            page_size, scale, temp_coef, temp_every, heads_per_chunk, k_pieces, v_pieces, window, keep_first, out_scale, sink,
+                            form, partial, gate};
+        if (dk <= 32) launch_tokens_values<1>(args, n_runs, grid, stream);
+        else if (dk <= 64) launch_tokens_values<2>(args, n_runs, grid, stream);
+        else if (dk <= 128) launch_tokens_values<4>(args, n_runs, grid, stream);
+        else launch_tokens_values<8>(args, n_runs, grid, stream);
+        if (partial && !unfinished) merge_runs_kernel<bf16_t><<<n_rows * H, std::min(MAX_VCHUNKS, (dv + WAVE - 1) / WAVE) * WAVE, 0, stream>>>((const float*)partial, (bf16_t*)out, n_runs, dv, out_scale,
+                                                                              (const float*)sink, H, gate);
     } else {
         static size_t allowed = 48 * 1024;
         if (lds > allowed && (allowed = lds))
@@ -1185,12 +1557,6 @@ NI_EXPORT int ni_bias_attention_mfma_rows(int dk, int dv, int one_pool) {
     if (dk % 16 || dv % 16 || dk < 16 || dv < 16 || dv > MAX_VCHUNKS * WAVE || (one_pool && dk != dv)) return 0;
     return mfma_lds_bytes(dk, dv, one_pool != 0) <= 160 * 1024 ? MROWS : 0;
 }
-
-struct MfmaArgs {
-    const void *qkv; int row_stride; const void *kpool, *vpool, *block_table; int table_width; const void *tiles, *positions, *bias;
-    int distances; void* out; int H, G, dk, dv, page_size; float scale, temp_coef; int temp_every, heads_per_chunk;
-    bool k_pieces, v_pieces; int window, keep_first; float out_scale; const void* sink; ScoreForm form; void* partial; Gate gate;
-};
 
 template <typename T, int QS, int DVB>
 static hipError_t launch_mfma(const MfmaArgs& a, dim3 grid, size_t lds, hipStream_t stream) {

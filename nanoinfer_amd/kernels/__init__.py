@@ -1203,7 +1203,7 @@ torch.backends.cudnn.allow_tf32 = False
 
 # sums onto the residual stream, routed experts, the gated delta rule, attention with a bias by distance
 from .stream import (BIAS_ATTENTION_MFMA_FROM, DELTA_RUN_FROM, EXPERTS_FEW_ROWS, add_rmsnormed, add_vector,  # noqa: E402,F401
-                     bias_attention, bias_attention_lib, bias_attention_mfma, bias_attention_mfma_rows, bias_attention_rows, bias_attention_runs, delta_rule, delta_rule_lib, embed_scaled, experts_act, experts_few,
+                     bias_attention, bias_attention_lib, bias_attention_mfma, bias_attention_mfma_rows, bias_attention_rows, bias_attention_runs, bias_attention_bf16_tokens, bias_attention_token_runs, delta_rule, delta_rule_lib, embed_scaled, experts_act, experts_few,
                      gated_side, kv_store, route_top, stream_add, stream_lib, embed_pair_hash, add_rows_vector, qk_norm_rope_store,
                      depth_mix, gate_heads, heads_apart, poly_norm, rmsnorm_cols, scale_, gate_rows, gather_pages, rows_to_pages,
                      post_norm, merge_maps, EXPERT_FORMS, ROUTE_SCORINGS, identity_experts, link_streams, LINK_STREAMS_MAX)

@@ -518,6 +518,21 @@ def bias_attention_runs(n_tiles: int, kv_heads: int, head_chunks: int, max_keys:
     return max(1, min(64, 2048 // (blocks * waves), max_keys // run_keys))
 
 
+TOKEN_RUN_KEYS = 128        # the same of the kernel for bfloat16, whose four wavefronts share a run's keys, 32 at a time
+TOKEN_WORKGROUPS = 1024     # ... and the workgroups that its runs aim for
+
+
+def bias_attention_bf16_tokens(dk: int, dv: int, dtype: torch.dtype) -> bool:
+    """Whether :func:`bias_attention` runs on the matrix cores for these sizes (bfloat16 alone)."""
+    return dtype == torch.bfloat16 and bool(bias_attention_lib().ni_bias_attention_bf16_tokens(int(dk), int(dv)))
+
+
+def bias_attention_token_runs(n_tiles: int, kv_heads: int, head_chunks: int, max_keys: int) -> int:
+    """:func:`bias_attention_runs` for that kernel: a workgroup's four wavefronts work on one run."""
+    blocks = max(1, n_tiles * kv_heads * head_chunks)
+    return max(1, min(64, TOKEN_WORKGROUPS // blocks, max_keys // TOKEN_RUN_KEYS))
+
+
 def bias_attention_rows() -> int:
     """Rows of (token, head) that one workgroup of the kernel takes."""
     return 16

@@ -235,7 +235,10 @@ class PagedSoftmax:
         chunk = self.extras["chunk"]
         reach = chunk if window is None else window + keep_first
         max_keys = ctx.max_context if reach is None else min(ctx.max_context, reach + self.tile_tokens + 128)
-        runs = K.bias_attention_runs(tiles.shape[0], self.G, chunks, max_keys, min(4, -(-rows // 4)))
+        if K.bias_attention_bf16_tokens(self.dk, self.dv, qkv.dtype):
+            runs = K.bias_attention_token_runs(tiles.shape[0], self.G, chunks, max_keys)
+        else:
+            runs = K.bias_attention_runs(tiles.shape[0], self.G, chunks, max_keys, min(4, -(-rows // 4)))
         ws = ctx.workspace(T * self.H * runs * (self.dv + 2)) if runs > 1 or not finish else None
         return K.bias_attention(qkv, kpool, vpool, block_table, tiles, ctx.positions, self.bias, out, self.H,
                                 self.scale, self.temp_coef, self.temp_every, self.heads_per_chunk, runs, ws, waves, window,
