@@ -637,7 +637,9 @@ def bias_attention(qkv: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, 
     ``maps`` m > 1: ``kpool`` rows hold m keys side by side, ``H`` counts the query heads of all maps, which come in the
     order [kv head][map][head of the group].  ``out`` None: the rows are left in ``workspace`` unfinished, every run by
     itself (:func:`merge_maps` takes them so), and the workspace is returned.  ``gate`` (rows, col, every): output channel j
-    of a token is multiplied by ``sigmoid(rows[t, col + j // every])``, ``rows`` float32 [T, wide]."""
+    of a token is multiplied by ``sigmoid(rows[t, col + j // every])``, ``rows`` float32 [T, wide].  Where
+    :func:`bias_attention_bf16_tokens` holds the kernel for the matrix cores runs (``waves`` then has no meaning: its four
+    wavefronts share the keys of a run)."""
     T, width = qkv.shape
     pages, G, ps, dk, dv = _map_sizes(kpool, vpool, maps)
     _gpu(qkv, "qkv")

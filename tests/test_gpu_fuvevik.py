@@ -272,7 +272,8 @@ def test_layer_by_layer_against_the_plain_stream(dtype):
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H,G,dk,dv,page,temp", [(6, 2, 16, 32, 8, (0.7, 19)), (4, 4, 32, 16, 16, (1.5, 64)), (3, 1, 24, 24, 4, (0.5, 1)),
                                                  (5, 5, 16, 16, 8, None), (8, 1, 112, 64, 8, (0.3, 100)), (2, 1, 20, 12, 8, (0.9, 33)),
-                                                 (16, 2, 64, 64, 16, (0.2, 128)), (3, 1, 48, 160, 8, (0.4, 63))])
+                                                 (16, 2, 64, 64, 16, (0.2, 128)), (3, 1, 48, 160, 8, (0.4, 63)),
+                                                 (20, 1, 32, 32, 4, (0.3, 40))])
 def test_far_keys_the_sink_and_the_query_factor_in_both_attention_kernels(H, G, dk, dv, page, temp, dtype):
     """The attention alone over scattered pages, with one key a query made to stand out: the first key, keys far back, at
     the edges of pages and of the kernels' tiles of 64, and the query's own.  The standing-out score is of the size of the
